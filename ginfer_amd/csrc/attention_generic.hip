@@ -76,7 +76,7 @@ __global__ __launch_bounds__(64 * GA_MAX_WAVES) void paged_attention_generic_ker
     const T* __restrict__ k_pages, const T* __restrict__ v_pages,
     const int32_t* __restrict__ block_table, int table_width,
     const int32_t* __restrict__ token_entry, const int32_t* __restrict__ positions, int tokens, int nh, int nkv,
-    int hd, int page_size, int window, float scale, int tq, int hpw, int min_run, const float* __restrict__ sinks) {
+    int hd, int page_size, int window, float scale, int tq, int hpw, int min_run, const HeadExtras ex) {
   extern __shared__ float lds[];
   const int group = nh / nkv, head_blocks = (group + hpw - 1) / hpw;     // hpw heads of a kv group to a workgroup
   const int waves = tq * hpw, threads = blockDim.x;        // wavefronts that compute; all threads load (see the launcher)
@@ -204,6 +204,7 @@ __global__ __launch_bounds__(64 * GA_MAX_WAVES) void paged_attention_generic_ker
         }
         for (; d < hd; ++d) dot = __builtin_fmaf(qr[d], kr[d], dot);
         s = dot * scale;
+        if (ex.cap > 0.f) s = ex.cap * tanhf(s / ex.cap);
       }
       const float m_new = fmaxf(m, wave_max(s));   // finite: every tile holds at least one valid key
       const float p = valid ? expf(s - m_new) : 0.f;
@@ -290,7 +291,8 @@ __global__ __launch_bounds__(64 * GA_MAX_WAVES) void paged_attention_generic_ker
   }
   if (!done) return;
   T* op = out + t * out_stride + (int64_t)h * hd;
-  const float inv = 1.0f / (sinks ? l + expf(sinks[h] - m) : l);     // a sink: a score with no value, in every sum
+  // a sink: a score with no value, in every sum; a gate: a factor of the head's result
+  const float inv = 1.0f / (ex.sinks ? l + expf(ex.sinks[h] - m) : l) * head_gate(ex, t, h);
 #pragma unroll
   for (int i = 0; i < MAX_HD / WAVE; ++i) {
     const int d = lane + i * WAVE;
@@ -443,7 +445,7 @@ __global__ __launch_bounds__(64 * (MA_MAX_COMPUTE + MA_LOADERS)) void paged_atte
     const T* __restrict__ k_pages, const T* __restrict__ v_pages,
     const int32_t* __restrict__ block_table, int table_width,
     const int32_t* __restrict__ token_entry, const int32_t* __restrict__ positions, int tokens, int nh, int nkv,
-    int page_size, int window, float scale, int tq, int hpw, const float* __restrict__ sinks) {
+    int page_size, int window, float scale, int tq, int hpw, const HeadExtras ex) {
   extern __shared__ float lds[];
   constexpr int hd = HD;
   constexpr int KS = HD + KPAD;                  // the layout of a tile in LDS: TileLoader
@@ -521,6 +523,7 @@ __global__ __launch_bounds__(64 * (MA_MAX_COMPUTE + MA_LOADERS)) void paged_atte
       continue;
     }
     const bool mine = live && tl >= run_begin && tl < run.end;
+    const float mul = ex.cap > 0.f ? 1.f : scale;
     done = done || mine;
     // one tile for this wavefront's tokens, its keys and values in LDS
     auto attend = [&](int tile, const float* k_s, const float* v_s) {
@@ -545,6 +548,12 @@ __global__ __launch_bounds__(64 * (MA_MAX_COMPUTE + MA_LOADERS)) void paged_atte
       // element r of block b: key 16 b + 4 kq + r of the tile, for this lane's token.  Where every token of the
       // wavefront sees all 64 keys (most tiles of a long prompt) nothing needs a mask: the same arithmetic without
       // the selects.
+      if (ex.cap > 0.f) {                                // capped scores: what follows multiplies them by one
+#pragma unroll
+        for (int b = 0; b < 4; ++b)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) s[b][r] = ex.cap * tanhf(s[b][r] * scale / ex.cap);
+      }
       const bool whole = __ballot(active && tile >= lo && tile + WAVE - 1 <= pos) == ~0ull;
       float m_new, alpha;
       if (whole) {
@@ -553,7 +562,7 @@ __global__ __launch_bounds__(64 * (MA_MAX_COMPUTE + MA_LOADERS)) void paged_atte
         for (int b = 0; b < 4; ++b)
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
-            s[b][r] = s[b][r] * scale;
+            s[b][r] = s[b][r] * mul;
             mx = fmaxf(mx, s[b][r]);
           }
         mx = fmaxf(mx, __shfl_xor(mx, 32, WAVE));
@@ -571,7 +580,7 @@ __global__ __launch_bounds__(64 * (MA_MAX_COMPUTE + MA_LOADERS)) void paged_atte
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
             const int c = tile + 16 * b + 4 * kq + r;
-            s[b][r] = (active && c >= lo && c <= pos) ? s[b][r] * scale : -INFINITY;
+            s[b][r] = (active && c >= lo && c <= pos) ? s[b][r] * mul : -INFINITY;
             mx = fmaxf(mx, s[b][r]);
           }
         mx = fmaxf(mx, __shfl_xor(mx, 32, WAVE));
@@ -643,7 +652,8 @@ __global__ __launch_bounds__(64 * (MA_MAX_COMPUTE + MA_LOADERS)) void paged_atte
   }
   if (!done) return;
   T* op = out + t * out_stride + (int64_t)h * hd;
-  const float inv = 1.0f / (sinks ? l + expf(sinks[h] - m) : l);     // a sink: a score with no value, in every sum
+  // a sink: a score with no value, in every sum; a gate: a factor of the head's result
+  const float inv = 1.0f / (ex.sinks ? l + expf(ex.sinks[h] - m) : l) * head_gate(ex, t, h);
 #pragma unroll
   for (int i = 0; i < NBLK; ++i)
 #pragma unroll
@@ -667,7 +677,7 @@ __global__ __launch_bounds__(64 * (HA_COMPUTE + HA_LOADERS)) void paged_attentio
     const T* __restrict__ k_pages, const T* __restrict__ v_pages,
     const int32_t* __restrict__ block_table, int table_width,
     const int32_t* __restrict__ token_entry, const int32_t* __restrict__ positions, int tokens, int nh, int nkv,
-    int page_size, int window, float scale, int min_run, const float* __restrict__ sinks) {
+    int page_size, int window, float scale, int min_run, const HeadExtras ex) {
   extern __shared__ float lds[];
   constexpr int KS = HD + KPAD;                  // the layout of a tile in LDS: TileLoader
   constexpr int NBLK = HD / 16;                  // blocks of 16 dimensions of the output
@@ -732,7 +742,9 @@ __global__ __launch_bounds__(64 * (HA_COMPUTE + HA_LOADERS)) void paged_attentio
     for (int r = 0; r < 4; ++r) {
       const int c = tile + 16 * wave + 4 * kq + r;
       valid[r] = live && c >= lo && c <= pos;
-      s[r] = valid[r] ? s[r] * scale : -INFINITY;
+      s[r] = s[r] * scale;
+      if (ex.cap > 0.f) s[r] = ex.cap * tanhf(s[r] / ex.cap);
+      s[r] = valid[r] ? s[r] : -INFINITY;
       mx = fmaxf(mx, s[r]);
     }
     mx = fmaxf(mx, __shfl_xor(mx, 32, WAVE));
@@ -779,7 +791,8 @@ __global__ __launch_bounds__(64 * (HA_COMPUTE + HA_LOADERS)) void paged_attentio
   }
   if (!live) return;
   T* op = out + t * out_stride + (int64_t)h * HD;
-  const float inv = 1.0f / (sinks ? l + expf(sinks[h] - m) : l);     // a sink: a score with no value, in every sum
+  // a sink: a score with no value, in every sum; a gate: a factor of the head's result
+  const float inv = 1.0f / (ex.sinks ? l + expf(ex.sinks[h] - m) : l) * head_gate(ex, t, h);
 #pragma unroll
   for (int i = 0; i < BPW; ++i) {
     const int blk = wave + HA_COMPUTE * i;
@@ -806,8 +819,9 @@ extern "C" int ga_paged_attention_generic(void* out, int64_t out_stride, const v
                                           const void* positions, int tokens, int nh, int nkv, int hd,
                                           int page_size, int window, float scale, int is_bf16,
                                           int tokens_per_workgroup, int few_tokens_workgroups,
-                                          int fill_workgroups, const void* sink_scores, hipStream_t stream) {
-  const float* sinks = (const float*)sink_scores;      // one score per head that every query sees beside its keys, or null
+                                          int fill_workgroups, const void* sink_scores, float cap, const void* gate,
+                                          int64_t gate_stride, float gate_scale, hipStream_t stream) {
+  const HeadExtras ex = {(const float*)sink_scores, cap, (const float*)gate, gate_stride, gate_scale};
   if (tokens <= 0) return 0;
   if (hd > MAX_HD || hd <= 0 || nkv <= 0 || nh % nkv != 0 || page_size <= 0) return -1;
   const int group = nh / nkv;
@@ -861,7 +875,7 @@ extern "C" int ga_paged_attention_generic(void* out, int64_t out_stride, const v
     hipLaunchKernelGGL((paged_attention_matrix_kernel<TT, VV, HH>), grid, block, lds, stream, (TT*)out, out_stride,  \
                        (const TT*)q, q_stride, (const TT*)k_pages, (const TT*)v_pages, (const int32_t*)block_table,  \
                        table_width, (const int32_t*)token_entry, (const int32_t*)positions, tokens, nh, nkv,          \
-                       page_size, window, scale, tq, hpw, sinks);                                                         \
+                       page_size, window, scale, tq, hpw, ex);                                                         \
   } while (0)
 #define LAUNCH_MATRIX_HD(TT, VV)                                                                                     \
   do {                                                                                                               \
@@ -913,7 +927,7 @@ extern "C" int ga_paged_attention_generic(void* out, int64_t out_stride, const v
     hipLaunchKernelGGL((paged_attention_heads_kernel<TT, VV, HH>), grid, block, lds, stream, (TT*)out, out_stride,   \
                        (const TT*)q, q_stride, (const TT*)k_pages, (const TT*)v_pages, (const int32_t*)block_table,  \
                        table_width, (const int32_t*)token_entry, (const int32_t*)positions, tokens, nh, nkv,          \
-                       page_size, window, scale, min_run, sinks);                                                         \
+                       page_size, window, scale, min_run, ex);                                                         \
   } while (0)
 #define LAUNCH_HEADS_HD(TT, VV)                                                                                      \
   do {                                                                                                               \
@@ -965,7 +979,7 @@ extern "C" int ga_paged_attention_generic(void* out, int64_t out_stride, const v
     hipLaunchKernelGGL((paged_attention_generic_kernel<TT, VV, PP>), grid, block, lds, stream, (TT*)out, out_stride, \
                        (const TT*)q, q_stride, (const TT*)k_pages, (const TT*)v_pages, (const int32_t*)block_table,  \
                        table_width, (const int32_t*)token_entry, (const int32_t*)positions, tokens, nh, nkv, hd,      \
-                       page_size, window, scale, tq, hpw, min_run, sinks);                                                \
+                       page_size, window, scale, tq, hpw, min_run, ex);                                                \
   } while (0)
   if (is_bf16) {
     if (wide && pipelined) LAUNCH(bf16_t, 8, true);

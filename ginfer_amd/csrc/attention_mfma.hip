@@ -31,6 +31,10 @@
 #include "common.h"
 #include "ginfer_amd.h"   // the entry points below are checked against their declarations
 
+// SOFT_CAP 1: the library for scores that are capped by a tanh; 0: the one for plain scores
+#ifndef SOFT_CAP
+#define SOFT_CAP 0
+#endif
 #ifndef HEAD_DIM
 #error "compile with -DHEAD_DIM=<head size>"
 #endif
@@ -68,6 +72,10 @@ typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2;
 // the bare v_exp_f32: arguments here are differences to a running maximum (<= 0, or -inf), for which the
 // library routine's extra steps for denormal results buy nothing
 __device__ __forceinline__ float fast_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
+// tanh(x) = 1 - 2 / (e^2x + 1) on the bare exponential and reciprocal: exact to some 1e-7, also at both ends
+__device__ __forceinline__ float fast_tanh(float x) {
+  return __builtin_fmaf(-2.f, __builtin_amdgcn_rcpf(fast_exp2(x * (2.f * LOG2E)) + 1.f), 1.f);
+}
 // A sink: a score that every query of a head sees beside its keys' and that has no value.  sinks: one score per head
 // (natural units; the maxima here are in units of log 2) or null.  The denominator l, relative to the maximum m, with
 // the sink's share added.
@@ -204,10 +212,15 @@ template <int NB>
 __device__ __forceinline__ void tile_softmax(bf16x8 (&pb)[NB], f32x4 (&s)[NB][2], f32x4 (&o)[NB][DB],
                                              float (&m)[NB], float (&l)[NB], const int (&cpos)[NB],
                                              const int (&clo)[NB], int full_lo, int full_hi, int k0, float scale,
-                                             int g) {
+                                             float cap, int g) {
   const bool interior = k0 >= full_lo && k0 + 31 <= full_hi;      // the same for the whole wavefront
 #pragma unroll
   for (int nb = 0; nb < NB; ++nb) {
+#if SOFT_CAP
+    // capped scores: tanh(q.k * cap), cap being scale / bound here; `scale` is then the bound (in units of log 2)
+#pragma unroll
+    for (int j = 0; j < 8; ++j) s[nb][j >> 2][j & 3] = fast_tanh(s[nb][j >> 2][j & 3] * cap);
+#endif
     if (!interior) {
       // The lane's key j is live where lo <= j <= hi: two subtractions here, none on the path without a mask.  The
       // scores are masked where they lie (a select: what was read for a dead key is dropped), so that the path
@@ -294,13 +307,13 @@ __device__ __forceinline__ void attend_one_tile(f32x4 (&o)[NB][DB], float (&m)[N
                                                 const bf16_t* __restrict__ v_pages,
                                                 const int32_t* __restrict__ bt, int table_width, int kvh, int nkv,
                                                 int ps_shift, int kv_min, int kv_max, int full_lo, int full_hi,
-                                                int k0, int k_refill, int k_lookup, float scale, int c, int g) {
+                                                int k0, int k_refill, int k_lookup, float scale, float cap, int c, int g) {
   f32x4 s[NB][2];
   tile_scores<NB>(s, kr, q);
   const bool refill_edge = k_refill < kv_min || k_refill + 31 > kv_max;
   if (k_refill >= 0) load_k_tile(kr, k_pages, pg, lk, kvh, nkv, ps_shift, k_refill, refill_edge, kv_min, kv_max, g);
   bf16x8 pb[NB];
-  tile_softmax<NB>(pb, s, o, m, l, cpos, clo, full_lo, full_hi, k0, scale, g);
+  tile_softmax<NB>(pb, s, o, m, l, cpos, clo, full_lo, full_hi, k0, scale, cap, g);
   tile_output<NB>(o, vr, pb, kv_min, kv_max, k0, g);
   if (k_refill >= 0) load_v_tile(vr, v_pages, pg, lk, kvh, nkv, ps_shift, k_refill, refill_edge, kv_min, kv_max, c);
   if (k_lookup >= 0) lookup_pages(pg, bt, table_width, ps_shift, k_lookup);
@@ -320,7 +333,7 @@ __device__ __forceinline__ void attend_tiles(f32x4 (&o)[NB][DB], float (&m)[NB],
                                              const bf16_t* __restrict__ v_pages,
                                              const int32_t* __restrict__ bt, int table_width, int kvh, int nkv,
                                              int ps_shift, int kv_min, int kv_max, int full_lo, int full_hi,
-                                             int tile_begin, int tile_end, int tile_stride, float scale) {
+                                             int tile_begin, int tile_end, int tile_stride, float scale, float cap) {
   static_assert(DEPTH == 1 || DEPTH == 2, "one or two sets of operand registers");
   const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
   // the same in every lane of the wavefront, by the callers' construction: said so, the loop and its branches
@@ -359,7 +372,7 @@ __device__ __forceinline__ void attend_tiles(f32x4 (&o)[NB][DB], float (&m)[NB],
         const int k_refill = k0 + DEPTH * tile_stride, k_lookup = k0 + 2 * DEPTH * tile_stride;
         attend_one_tile<NB>(o, m, l, q, cpos, clo, kr[d], vr[d], pg[d], lk, k_pages, v_pages, bt, table_width, kvh,
                             nkv, ps_shift, kv_min, kv_max, full_lo, full_hi, k0, k_refill < tile_end ? k_refill : -1,
-                            k_lookup < tile_end ? k_lookup : -1, scale, c, g);
+                            k_lookup < tile_end ? k_lookup : -1, scale, cap, c, g);
       }
     }
   }
@@ -407,7 +420,7 @@ __global__ __launch_bounds__(64 * DEC_WAVES) void attn_decode_split_kernel(
     const bf16_t* __restrict__ q, int64_t q_stride, const bf16_t* __restrict__ k_pages,
     const bf16_t* __restrict__ v_pages, const int32_t* __restrict__ block_table, int table_width,
     const int4* __restrict__ decode_info, int nh, int nkv, int head_blocks, int ps_shift, int window,
-    float scale, int split_keys, int num_splits, const float* __restrict__ sinks) {
+    float scale, int split_keys, int num_splits, const HeadExtras ex) {
   __shared__ float o_s[DEC_WAVES][HD][17];
   __shared__ float m_s[DEC_WAVES][16], l_s[DEC_WAVES][16], mx_s[16], lsum_s[16];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c = lane & 15, g = lane >> 4;
@@ -433,7 +446,7 @@ __global__ __launch_bounds__(64 * DEC_WAVES) void attn_decode_split_kernel(
     const int32_t* bt = block_table + (int64_t)__builtin_amdgcn_readfirstlane(info.z) * table_width;
     // every live column of a decode wavefront sees the same keys: lo..pos
     attend_tiles<1, DECODE_DEPTH>(o, m, l, qr, cpos, clo, k_pages, v_pages, bt, table_width, kvh, nkv, ps_shift, lo,
-                                  pos, lo, pos, begin + 32 * wave, end, 32 * DEC_WAVES, scale);
+                                  pos, lo, pos, begin + 32 * wave, end, 32 * DEC_WAVES, scale, ex.cap);
     finish_sums<1>(l);
   }
   // the wavefronts' states meet: common max, rescaled sums and outputs added in wavefront order
@@ -476,7 +489,7 @@ __global__ __launch_bounds__(64 * DEC_WAVES) void attn_decode_split_kernel(
     for (int w = 0; w < DEC_WAVES; ++w) acc += o_s[w][d][cc];
     if (num_splits == 1) {
       const int hh = kvh * group + hb * 16 + cc;
-      out[(int64_t)t * out_stride + (int64_t)hh * HD + d] = f32_to_bf16(acc / sink_sum(lsum_s[cc], mx_s[cc], sinks, hh));
+      out[(int64_t)t * out_stride + (int64_t)hh * HD + d] = f32_to_bf16(acc / sink_sum(lsum_s[cc], mx_s[cc], ex.sinks, hh) * head_gate(ex, t, hh));
     } else {
       const int64_t slot = slot_base + (int64_t)cc * num_splits;
       part_o[slot * HD + d] = acc;
@@ -497,7 +510,7 @@ template <int EARLY>
 __global__ __launch_bounds__(64) void attn_decode_combine_kernel(
     bf16_t* __restrict__ out, int64_t out_stride, const float* __restrict__ part_o,
     const float* __restrict__ part_ml, const int4* __restrict__ decode_info, int nh, int num_splits,
-    const float* __restrict__ sinks) {
+    const HeadExtras ex) {
   __shared__ float w_s[MAX_SPLITS];
   const int ti = blockIdx.x, head = blockIdx.y, lane = threadIdx.x;
   const int64_t base = ((int64_t)ti * nh + head) * num_splits;
@@ -524,7 +537,7 @@ __global__ __launch_bounds__(64) void attn_decode_combine_kernel(
   }
   total = wave_sum(total);
   __syncthreads();
-  const float inv = 1.f / sink_sum(total, mx, sinks, head);
+  const float inv = 1.f / sink_sum(total, mx, ex.sinks, head) * head_gate(ex, row, head);
   bf16_t* op = out + (int64_t)row * out_stride + (int64_t)head * HD;
   if (EARLY > 0) {
 #pragma unroll
@@ -577,7 +590,7 @@ template <int NB>
 __device__ __forceinline__ void write_rows(const f32x4 (&o)[NB][DB], const float (&m)[NB], const float (&l)[NB],
                                            bf16_t* __restrict__ out, int64_t out_stride, float* __restrict__ part_o,
                                            float* __restrict__ part_ml, const KeyPart& kp, int row0, int rows, int head,
-                                           int nh, int c, int g, const float* __restrict__ sinks) {
+                                           int nh, int c, int g, const HeadExtras& ex) {
 #pragma unroll
   for (int nb = 0; nb < NB; ++nb) {
     const int j = nb * 16 + c;
@@ -593,7 +606,7 @@ __device__ __forceinline__ void write_rows(const f32x4 (&o)[NB][DB], const float
       }
       continue;
     }
-    const float inv = 1.f / sink_sum(l[nb], m[nb], sinks, head);
+    const float inv = 1.f / sink_sum(l[nb], m[nb], ex.sinks, head) * head_gate(ex, row0 + j, head);
     bf16_t* op = out + (int64_t)(row0 + j) * out_stride + (int64_t)head * HD + g * 4;
 #pragma unroll
     for (int db = 0; db < DB; ++db) {
@@ -617,7 +630,7 @@ __global__ __launch_bounds__(64 * PREFILL_WAVES) void attn_prefill_kernel(
     const int32_t* __restrict__ block_table, int table_width, const int32_t* __restrict__ tiles, int nh,
     int nkv, int head_blocks, int hpw, int splits, int ps_shift, int window, float scale,
     const int32_t* __restrict__ parts, float* __restrict__ part_o, float* __restrict__ part_ml,
-    const float* __restrict__ sinks) {
+    const HeadExtras ex) {
   extern __shared__ float lds[];          // [hpw][splits-1][NB] x { o[HD][17], m[16], l[16] }
   constexpr int STATE = HD * 17 + 32;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c = lane & 15, g = lane >> 4;
@@ -663,7 +676,7 @@ __global__ __launch_bounds__(64 * PREFILL_WAVES) void attn_prefill_kernel(
     attend_tiles<NB, PREFILL_DEPTH>(o, m, l, qr, cpos, clo, k_pages, v_pages,
                                     block_table + (int64_t)__builtin_amdgcn_readfirstlane(entry) * table_width,
                                     table_width, kvh, nkv, ps_shift, kv_min, kv_max, full_lo, pos0,
-                                    kp.begin + 32 * split, kp.end, 32 * splits, scale);
+                                    kp.begin + 32 * split, kp.end, 32 * splits, scale, ex.cap);
     finish_sums<NB>(l);
   }
   if (splits > 1) {
@@ -708,7 +721,7 @@ __global__ __launch_bounds__(64 * PREFILL_WAVES) void attn_prefill_kernel(
   } else if (!head_ok) {
     return;
   }
-  write_rows<NB>(o, m, l, out, out_stride, part_o, part_ml, kp, row0, rows, head, nh, c, g, sinks);
+  write_rows<NB>(o, m, l, out, out_stride, part_o, part_ml, kp, row0, rows, head, nh, c, g, ex);
 }
 
 // ----------------------------------------------------------------------------- prefill, operands through LDS
@@ -785,7 +798,7 @@ __global__ __launch_bounds__(64 * PREFILL_WAVES) void attn_prefill_shared_kernel
     const int32_t* __restrict__ block_table, int table_width, const int32_t* __restrict__ tiles, int nh,
     int nkv, int head_blocks, int hpw, int splits, int ps_shift, int window, float scale,
     const int32_t* __restrict__ parts, float* __restrict__ part_o, float* __restrict__ part_ml,
-    const float* __restrict__ sinks) {
+    const HeadExtras ex) {
   static_assert(STAGES == 2 || STAGES == 3, "two or three stages");
   extern __shared__ __attribute__((aligned(16))) unsigned char ring[];
   float* lds = reinterpret_cast<float*>(ring);      // after the loop: [hpw][splits-1][NB] x { o[HD][17], m[16], l[16] }
@@ -888,7 +901,7 @@ __global__ __launch_bounds__(64 * PREFILL_WAVES) void attn_prefill_shared_kernel
         f32x4 s[NB][2];
         tile_scores<NB>(s, kr, qr);
         bf16x8 pb[NB];
-        tile_softmax<NB>(pb, s, o, m, l, cpos, clo, full_lo, pos0, k0, scale, g);
+        tile_softmax<NB>(pb, s, o, m, l, cpos, clo, full_lo, pos0, k0, scale, ex.cap, g);
         tile_output<NB>(o, vr, pb, kv_min, kv_max, k0, g);
       }
     }
@@ -939,9 +952,21 @@ __global__ __launch_bounds__(64 * PREFILL_WAVES) void attn_prefill_shared_kernel
   } else if (!head_ok) {
     return;
   }
-  write_rows<NB>(o, m, l, out, out_stride, part_o, part_ml, kp, row0, rows, head, nh, c, g, sinks);
+  write_rows<NB>(o, m, l, out, out_stride, part_o, part_ml, kp, row0, rows, head, nh, c, g, ex);
 }
 #endif
+
+// What the kernels take as scale and cap: with capped scores the bound is the scale of the softmax, and scale / bound goes
+// into the tanh.  false: this library was not built for such scores (or for none but such).
+static bool bound_scores(float& scale, HeadExtras& ex) {
+  if ((ex.cap > 0.f) != (SOFT_CAP != 0)) return false;
+  if (ex.cap > 0.f) {
+    const float bound = ex.cap;
+    ex.cap = scale / bound;
+    scale = bound;
+  }
+  return true;
+}
 
 extern "C" int ga_attn_head_dim() { return HD; }
 // rows of a prefill tile: 16 or (head sizes up to 128) 32
@@ -954,7 +979,8 @@ extern "C" int ga_attn_decode(void* out, int64_t out_stride, const void* q, int6
                               const void* v_pages, const void* block_table, int table_width,
                               const void* decode_info, int n_tokens, int nh, int nkv, int page_size, int window, float scale,
                               int split_keys, int num_splits, void* workspace_o, void* workspace_ml,
-                              const void* sinks, hipStream_t stream) {
+                              const void* sinks, float cap, const void* gate, int64_t gate_stride, float gate_scale,
+                              hipStream_t stream) {
   if (n_tokens <= 0) return 0;
   if (nkv <= 0 || nh % nkv) return -1;
   int ps_shift = 0;
@@ -964,18 +990,20 @@ extern "C" int ga_attn_decode(void* out, int64_t out_stride, const void* q, int6
   const int group = nh / nkv, head_blocks = (group + 15) / 16;
   if ((int64_t)nkv * head_blocks > 65535) return -4;
   if (num_splits > MAX_SPLITS) return -5;
+  HeadExtras ex = {(const float*)sinks, cap, (const float*)gate, gate_stride, gate_scale};
+  if (!bound_scores(scale, ex)) return -20;
   dim3 grid(n_tokens, nkv * head_blocks, num_splits);
   hipLaunchKernelGGL(attn_decode_split_kernel, grid, dim3(64 * DEC_WAVES), 0, stream, (bf16_t*)out, out_stride,
                      (float*)workspace_o, (float*)workspace_ml, (const bf16_t*)q, q_stride,
                      (const bf16_t*)k_pages, (const bf16_t*)v_pages, (const int32_t*)block_table, table_width,
                      (const int4*)decode_info, nh, nkv, head_blocks, ps_shift, window, scale * LOG2E, split_keys,
-                     num_splits, (const float*)sinks);
+                     num_splits, ex);
   int rc = GA_CHECK_LAUNCH();
   if (rc || num_splits == 1) return rc;
 #define COMBINE(EARLY)                                                                                       \
   hipLaunchKernelGGL(attn_decode_combine_kernel<EARLY>, dim3(n_tokens, nh), dim3(64), 0, stream, (bf16_t*)out, \
                      out_stride, (const float*)workspace_o, (const float*)workspace_ml,                        \
-                     (const int4*)decode_info, nh, num_splits, (const float*)sinks)
+                     (const int4*)decode_info, nh, num_splits, ex)
   if (num_splits <= 8) COMBINE(8);
   else if (num_splits <= 16) COMBINE(16);
   else if (num_splits <= 32) COMBINE(32);
@@ -988,7 +1016,7 @@ static int attn_prefill_tiles(void* out, int64_t out_stride, const void* q, int6
                               const void* v_pages, const void* block_table, int table_width, const void* tiles,
                               int n_tiles, int tile_rows, int nh, int nkv, int page_size, int window, float scale,
                               int fill_workgroups, int prefer_workgroups, const void* parts, void* part_o,
-                              void* part_ml, const void* sinks, hipStream_t stream);
+                              void* part_ml, const HeadExtras& ex, hipStream_t stream);
 
 // parts: null, or for every tile int32 x 4 = (first key, end of keys, index of the tile's first row among the rows that
 // come in parts, part + (number of parts << 16)); a tile whose keys are dealt to several workgroups stands in `tiles` once
@@ -999,18 +1027,21 @@ extern "C" int ga_attn_prefill(void* out, int64_t out_stride, const void* q, int
                                int table_width, const void* tiles, int n_tiles, int tile_rows, int nh, int nkv,
                                int page_size, int window, float scale, int fill_workgroups, int prefer_workgroups,
                                const void* parts, const void* part_rows, int n_part_rows, int num_parts, void* part_o,
-                               void* part_ml, const void* sinks, hipStream_t stream) {
+                               void* part_ml, const void* sinks, float cap, const void* gate, int64_t gate_stride,
+                               float gate_scale, hipStream_t stream) {
   if (n_tiles <= 0) return 0;
+  HeadExtras ex = {(const float*)sinks, cap, (const float*)gate, gate_stride, gate_scale};
+  if (!bound_scores(scale, ex)) return -20;
   if (nkv <= 0 || nh % nkv) return -1;
   if (parts && (n_part_rows <= 0 || num_parts < 2 || num_parts > 8 || !part_rows || !part_o || !part_ml)) return -8;
   if (!parts) n_part_rows = 0;
   int rc = attn_prefill_tiles(out, out_stride, q, q_stride, k_pages, v_pages, block_table, table_width, tiles, n_tiles,
                               tile_rows, nh, nkv, page_size, window, scale, fill_workgroups, prefer_workgroups, parts, part_o,
-                              part_ml, sinks, stream);
+                              part_ml, ex, stream);
   if (rc || n_part_rows == 0) return rc;
   hipLaunchKernelGGL(attn_decode_combine_kernel<8>, dim3(n_part_rows, nh), dim3(64), 0, stream, (bf16_t*)out, out_stride,
                      (const float*)part_o, (const float*)part_ml, (const int4*)part_rows, nh, num_parts,
-                     (const float*)sinks);
+                     ex);
   return GA_CHECK_LAUNCH();
 }
 
@@ -1018,7 +1049,7 @@ static int attn_prefill_tiles(void* out, int64_t out_stride, const void* q, int6
                               const void* k_pages, const void* v_pages, const void* block_table,
                               int table_width, const void* tiles, int n_tiles, int tile_rows, int nh, int nkv,
                               int page_size, int window, float scale, int fill_workgroups, int prefer_workgroups,
-                              const void* parts, void* part_o, void* part_ml, const void* sinks, hipStream_t stream) {
+                              const void* parts, void* part_o, void* part_ml, const HeadExtras& ex, hipStream_t stream) {
   if (tile_rows != 16 && tile_rows != 16 * PREFILL_NB) return -6;
   int ps_shift = 0;
   while ((1 << ps_shift) < page_size) ++ps_shift;
@@ -1062,7 +1093,7 @@ static int attn_prefill_tiles(void* out, int64_t out_stride, const void* q, int6
                        out_stride, (const bf16_t*)q, q_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages, \
                        (const int32_t*)block_table, table_width, (const int32_t*)tiles, nh, nkv, head_blocks,  \
                        heads, streams, ps_shift, window, scale * LOG2E, (const int32_t*)parts, (float*)part_o, \
-                       (float*)part_ml, (const float*)sinks);                                                  \
+                       (float*)part_ml, ex);                                                  \
   } while (0)
       if (nb == 1) {
         if (stages == 3) LAUNCH_SHARED(1, 3); else LAUNCH_SHARED(1, 2);
@@ -1093,7 +1124,7 @@ static int attn_prefill_tiles(void* out, int64_t out_stride, const void* q, int6
                      (const bf16_t*)q, q_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages,           \
                      (const int32_t*)block_table, table_width, (const int32_t*)tiles, nh, nkv, head_blocks, \
                      hpw, splits, ps_shift, window, scale * LOG2E, (const int32_t*)parts, (float*)part_o,   \
-                     (float*)part_ml, (const float*)sinks)
+                     (float*)part_ml, ex)
   if (lds > 48 * 1024) {                     // more dynamic LDS than the default limit: ask for it
     const void* fn = nb == 1 ? (const void*)attn_prefill_kernel<1> : (const void*)attn_prefill_kernel<PREFILL_NB>;
     if (hipFuncSetAttribute(fn, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return -7;

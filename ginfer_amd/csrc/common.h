@@ -68,6 +68,24 @@ __host__ __device__ __forceinline__ int first_visible_key(int pos, int window) {
   return 0;
 }
 
+// What the attention kernels know of a head beyond its keys.  sinks: null, or one score per head that every query sees beside
+// its keys' and that has no value; cap: 0, or the bound of scores that are capped (score <- cap * tanh(score / cap)); gate:
+// null, or float rows (row stride gate_stride) with a number per head whose sigmoid, times gate_scale, multiplies the head's
+// result.
+struct HeadExtras {
+  const float* sinks;
+  float cap;
+  const float* gate;
+  int64_t gate_stride;
+  float gate_scale;
+};
+
+// the factor of head `head`'s result at row `row` of the step (1 without a gate)
+__device__ __forceinline__ float head_gate(const HeadExtras& ex, int64_t row, int head) {
+  if (ex.gate == nullptr) return 1.f;
+  return ex.gate_scale / (1.f + expf(-ex.gate[row * ex.gate_stride + head]));
+}
+
 #define GA_CHECK_LAUNCH() ((int)hipGetLastError())
 
 // Page and place in the page of a cache slot (slot >= 0).  Page sizes are powers of two nearly always: then a shift,

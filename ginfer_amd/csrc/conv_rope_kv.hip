@@ -3,7 +3,8 @@
 // (a workgroup per token and head)
 //   c[ch]  = sum_j w[ch, j] * u[t - taps + 1 + j, ch]     (u: the projection's rows; those before the step's tokens come
 //                                                           from per-request state, zeros before the sequence's start)
-//   q, k:    optionally divided by the root mean square of the token's whole q (k) projection, times a gain per channel
+//   q, k:    optionally divided by the root mean square of the token's whole q (k) projection, times a gain per channel;
+//            or every head by its own root mean square, times a gain per coordinate that the heads share (q's and k's own)
 //   q, k:    the first rotary_dim coordinates of every head turned by the position's angle (pairs i, i + rotary_dim/2)
 //   q   ->   out[t, head * padded + d]                      (heads padded with zeros to the width the attention takes)
 //   k   ->   k_pages[page, kv head, place, d],   v -> v_pages[page, kv head, d, place]   (padded alike)
@@ -26,7 +27,8 @@ __global__ __launch_bounds__(CR_HEAD_THREADS) void conv_rope_kv_kernel(
     const int32_t* __restrict__ q_start, const int32_t* __restrict__ positions, const float* __restrict__ cos_t,
     const float* __restrict__ sin_t, const int64_t* __restrict__ slot_mapping, T* __restrict__ k_pages, T* __restrict__ v_pages,
     int nh, int nkv, int hd, int vd, int padded, int rotary_dim, int taps, int page_size, int write_kv,
-    const float* __restrict__ row_scale, const float* __restrict__ gain) {
+    const float* __restrict__ row_scale, const float* __restrict__ gain, int64_t stride, float head_eps) {
+  __shared__ float scratch[CR_HEAD_THREADS / WAVE];
   __shared__ float head[CR_HEAD_THREADS];              // the head's convolved channels
   const int64_t t = blockIdx.x;
   const int h = blockIdx.y, d = threadIdx.x;
@@ -41,7 +43,7 @@ __global__ __launch_bounds__(CR_HEAD_THREADS) void conv_rope_kv_kernel(
   if (d < own) {
     const int c = first + d;
     if (w == nullptr) {
-      acc = Num<U>::ld(proj + t * width + c);
+      acc = Num<U>::ld(proj + t * stride + c);
     } else {
       const int e = token_entry[t];
       const int local = (int)t - cu[e];
@@ -50,7 +52,7 @@ __global__ __launch_bounds__(CR_HEAD_THREADS) void conv_rope_kv_kernel(
       for (int j = 0; j < taps; ++j) {
         const int back = taps - 1 - j;
         float v;
-        if (local - back >= 0) v = Num<U>::ld(proj + (t - back) * width + c);
+        if (local - back >= 0) v = Num<U>::ld(proj + (t - back) * stride + c);
         else if (fresh) v = 0.f;
         else v = st[(int64_t)(taps - 1 + local - back) * width + c];
         acc += w[(int64_t)c * taps + j] * v;
@@ -59,6 +61,17 @@ __global__ __launch_bounds__(CR_HEAD_THREADS) void conv_rope_kv_kernel(
   }
   // a norm over the whole projection of q (and of k): the row's factor from the launch before, a gain per channel
   if (row_scale != nullptr && !(!is_q && !is_k) && d < own) acc = acc * row_scale[t * 2 + (is_k ? 1 : 0)] * gain[first + d];
+  // a norm per head over its own coordinates; gain [2][hd]: q's, then k's
+  if (head_eps >= 0.f && (is_q || is_k)) {
+    float ss = wave_sum(acc * acc);                    // (acc is zero from a head's own width on)
+    if (blockDim.x > WAVE) {
+      if ((d & (WAVE - 1)) == 0) scratch[d / WAVE] = ss;
+      __syncthreads();
+      ss = 0.f;
+      for (int i = 0; i < (int)blockDim.x / WAVE; ++i) ss += scratch[i];
+    }
+    if (d < hd) acc = acc / sqrtf(ss / (float)hd + head_eps) * gain[(is_k ? hd : 0) + d];
+  }
   const bool rotate = (is_q || is_k) && cos_t != nullptr;
   if (rotate) {
     head[d] = acc;
@@ -86,10 +99,10 @@ __global__ __launch_bounds__(CR_HEAD_THREADS) void conv_rope_kv_kernel(
 // heads.  A workgroup a token; every thread's partial sum and the workgroup's sum in an order that depends on the sizes alone.
 template <typename U>
 __global__ __launch_bounds__(CR_THREADS) void projection_rms_kernel(float* __restrict__ row_scale, const U* __restrict__ proj,
-                                                                     int width, int q_width, int k_width, float eps) {
+                                                                     int64_t stride, int q_width, int k_width, float eps) {
   __shared__ float scratch[CR_THREADS / WAVE];
   const int64_t t = blockIdx.x;
-  const U* row = proj + t * width;
+  const U* row = proj + t * stride;
   float sq = 0.f, sk = 0.f;
   for (int i = threadIdx.x; i < q_width; i += CR_THREADS) { const float v = Num<U>::ld(row + i); sq = fmaf(v, v, sq); }
   for (int i = threadIdx.x; i < k_width; i += CR_THREADS) { const float v = Num<U>::ld(row + q_width + i); sk = fmaf(v, v, sk); }
@@ -107,7 +120,8 @@ template <typename T>
 __global__ __launch_bounds__(CR_THREADS) void conv_state_update_kernel(float* __restrict__ state, const T* __restrict__ proj,
                                                                         const int64_t* __restrict__ slots,
                                                                         const int32_t* __restrict__ cu,
-                                                                        const int32_t* __restrict__ q_start, int width, int taps) {
+                                                                        const int32_t* __restrict__ q_start, int width, int taps,
+                                                                        int64_t stride) {
   const int e = blockIdx.x;
   const int first = cu[e], n = cu[e + 1] - first;
   if (n <= 0) return;
@@ -117,7 +131,7 @@ __global__ __launch_bounds__(CR_THREADS) void conv_state_update_kernel(float* __
     for (int k = 0; k < taps - 1; ++k) {
       const int local = n - (taps - 1) + k;
       float v;
-      if (local >= 0) v = Num<T>::ld(proj + (int64_t)(first + local) * width + c);
+      if (local >= 0) v = Num<T>::ld(proj + (int64_t)(first + local) * stride + c);
       else if (fresh) v = 0.f;
       else v = st[(int64_t)(n + k) * width + c];
       st[(int64_t)k * width + c] = v;
@@ -130,7 +144,7 @@ extern "C" int ga_conv_rope_kv(void* q_out, const void* proj, const void* w, voi
                                const void* cos_t, const void* sin_t, const void* slot_mapping, void* k_pages, void* v_pages,
                                int tokens, int entries, int nh, int nkv, int hd, int vd, int padded, int rotary_dim, int taps,
                                int page_size, int write_kv, int update_state, int is_bf16, int proj_bf16, void* row_scale,
-                               const void* gain, float norm_eps, hipStream_t stream) {
+                               const void* gain, float norm_eps, int64_t stride, float head_eps, hipStream_t stream) {
   if (tokens <= 0) return 0;
   if (nh <= 0 || nkv <= 0 || hd <= 0 || vd <= 0 || padded < hd || padded < vd || page_size <= 0) return -1;
   if (taps < 1 || taps > CR_MAX_TAPS || (w == nullptr && taps != 1)) return -2;
@@ -139,7 +153,9 @@ extern "C" int ga_conv_rope_kv(void* q_out, const void* proj, const void* w, voi
   if (write_kv && (!slot_mapping || !k_pages || !v_pages)) return -5;
   const int width = (nh + nkv) * hd + nkv * vd;
   if (padded > CR_HEAD_THREADS) return -6;
-  if ((row_scale != nullptr) != (gain != nullptr) || (row_scale != nullptr && taps != 1)) return -9;
+  const bool by_head = head_eps >= 0.f;
+  if ((row_scale != nullptr || by_head) != (gain != nullptr) || (row_scale != nullptr && (taps != 1 || by_head))) return -9;
+  if (stride < width) return -10;
   if (nh + 2 * nkv > 65535) return -7;
   int threads = 64;
   while (threads < padded) threads *= 2;
@@ -147,13 +163,13 @@ extern "C" int ga_conv_rope_kv(void* q_out, const void* proj, const void* w, voi
   do {                                                                                                                 \
     if (row_scale != nullptr)                                                                                          \
       hipLaunchKernelGGL(projection_rms_kernel<U>, dim3(tokens), dim3(CR_THREADS), 0, stream, (float*)row_scale,       \
-                         (const U*)proj, width, nh * hd, nkv * hd, norm_eps);                                          \
+                         (const U*)proj, stride, nh * hd, nkv * hd, norm_eps);                                          \
     hipLaunchKernelGGL((conv_rope_kv_kernel<T, U>), dim3(tokens, nh + 2 * nkv), dim3(threads), 0, stream, (T*)q_out,   \
                        (const U*)proj, (const float*)w, (const float*)state, (const int64_t*)slots,                    \
                        (const int32_t*)token_entry, (const int32_t*)cu, (const int32_t*)q_start,                       \
                        (const int32_t*)positions, (const float*)cos_t, (const float*)sin_t,                            \
                        (const int64_t*)slot_mapping, (T*)k_pages, (T*)v_pages, nh, nkv, hd, vd, padded, rotary_dim,    \
-                       taps, page_size, write_kv, (const float*)row_scale, (const float*)gain);                        \
+                       taps, page_size, write_kv, (const float*)row_scale, (const float*)gain, stride, head_eps);      \
     int rc = GA_CHECK_LAUNCH();                                                                                        \
     if (rc) return rc;                                                                                                 \
     if (update_state && taps > 1 && entries > 0) {                                                                     \
@@ -161,7 +177,7 @@ extern "C" int ga_conv_rope_kv(void* q_out, const void* proj, const void* w, voi
       if (cols > 64) cols = 64;                                                                                        \
       hipLaunchKernelGGL(conv_state_update_kernel<U>, dim3(entries, cols), dim3(CR_THREADS), 0, stream, (float*)state, \
                          (const U*)proj, (const int64_t*)slots, (const int32_t*)cu, (const int32_t*)q_start, width,    \
-                         taps);                                                                                        \
+                         taps, stride);                                                                                        \
     }                                                                                                                  \
   } while (0)
   if (!is_bf16 && proj_bf16) return -8;

@@ -12,7 +12,7 @@
 // steps, nor on what else is in the batch.
 // gla_decay: a = sigmoid(z)^(1/tau), z = A2 (low) + b (A2 handed over transposed), `low` being the rows of a narrow projection (32-bit), as
 //   exp(-softplus(-z) / tau), all in 32-bit.
-// head_norm_gate: out[t, h, :] = o[t, h, :] / sqrt(mean(o[t, h, :]^2) + eps) (* weight[:]) (* silu(gate[t, h, :]), or * sigmoid of it).
+// head_norm_gate (times out_scale; weight: shared by the heads, or every head its own): out[t, h, :] = o[t, h, :] / sqrt(mean(o[t, h, :]^2) + eps) (* weight[:]) (* silu(gate[t, h, :]), or * sigmoid of it).
 // silu_inputs: the recurrence reads silu(q), silu(k), silu(v) in place of the projection's numbers.
 #include "common.h"
 #include "ginfer_amd.h"
@@ -191,7 +191,8 @@ __global__ __launch_bounds__(DS_THREADS) void head_norm_gate_kernel(T* __restric
                                                                      const float* __restrict__ weight,
                                                                      const float* __restrict__ gate, int64_t gate_stride,
                                                                      int64_t rows, int heads, int vdim, float eps,
-                                                                     int sigmoid_gate) {
+                                                                     int sigmoid_gate, int64_t out_stride, int weight_stride,
+                                                                     float out_scale) {
   const int64_t row = (int64_t)blockIdx.x * (DS_THREADS / WAVE) + threadIdx.x / WAVE;
   if (row >= rows) return;
   const int lane = threadIdx.x % WAVE;
@@ -205,12 +206,12 @@ __global__ __launch_bounds__(DS_THREADS) void head_norm_gate_kernel(T* __restric
   const float* g = gate ? gate + t * gate_stride + (int64_t)h * vdim : nullptr;
   for (int i = lane; i < vdim; i += WAVE) {
     float y = p[i] / rms;
-    if (weight) y *= weight[i];
+    if (weight) y *= weight[h * weight_stride + i];
     if (g) {
       const float z = g[i];
       y *= (sigmoid_gate ? 1.0f : z) / (1.0f + expf(-z));
     }
-    Num<T>::st(out + row * vdim + i, y);
+    Num<T>::st(out + t * out_stride + (int64_t)h * vdim + i, y * out_scale);
   }
 }
 
@@ -219,7 +220,8 @@ template <typename T>
 __global__ __launch_bounds__(DS_THREADS) void wide_norm_gate_kernel(T* __restrict__ out, const float* __restrict__ x,
                                                                      const float* __restrict__ weight,
                                                                      const float* __restrict__ gate, int64_t gate_stride,
-                                                                     int width, float eps, int sigmoid_gate) {
+                                                                     int width, float eps, int sigmoid_gate, int64_t out_stride, int weight_stride,
+                                                                     float out_scale) {
   __shared__ float scratch[DS_THREADS / WAVE];
   const int64_t t = blockIdx.x;
   const float* p = x + t * width;
@@ -235,7 +237,7 @@ __global__ __launch_bounds__(DS_THREADS) void wide_norm_gate_kernel(T* __restric
       const float z = g[i];
       y *= (sigmoid_gate ? 1.0f : z) / (1.0f + expf(-z));
     }
-    Num<T>::st(out + t * width + i, y);
+    Num<T>::st(out + t * out_stride + i, y * out_scale);
   }
 }
 
@@ -245,7 +247,8 @@ template <typename T, int PER>
 __global__ __launch_bounds__(DS_THREADS) void wide_norm_gate_rows_kernel(T* __restrict__ out, const float* __restrict__ x,
                                                                           const float* __restrict__ weight,
                                                                           const float* __restrict__ gate, int64_t gate_stride,
-                                                                          int width, float eps, int sigmoid_gate) {
+                                                                          int width, float eps, int sigmoid_gate, int64_t out_stride, int weight_stride,
+                                                                     float out_scale) {
   __shared__ float scratch[DS_THREADS / WAVE];
   const int64_t t = blockIdx.x;
   float4 xv[PER], wv[PER], gv[PER];
@@ -285,7 +288,7 @@ __global__ __launch_bounds__(DS_THREADS) void wide_norm_gate_rows_kernel(T* __re
         float y = e[k] / rms;
         if (weight) y *= w4[k];
         if (gate) y *= (sigmoid_gate ? 1.0f : g4[k]) / (1.0f + expf(-g4[k]));
-        Num<T>::st(out + t * width + i + k, y);
+        Num<T>::st(out + t * out_stride + i + k, y * out_scale);
       }
     }
   }
@@ -331,14 +334,14 @@ extern "C" int ga_gla_decay(void* decay, const void* low, int64_t low_stride, co
 
 extern "C" int ga_head_norm_gate(void* out, const void* x, const void* weight, const void* gate, int64_t gate_stride,
                                  int64_t tokens, int heads, int vdim, float eps, int out_bf16, int sigmoid_gate,
-                                 hipStream_t stream) {
+                                 int64_t out_stride, int weight_stride, float out_scale, hipStream_t stream) {
   if (tokens <= 0) return 0;
-  if (vdim <= 0 || heads <= 0) return -1;
+  if (vdim <= 0 || heads <= 0 || out_stride < (int64_t)heads * vdim || weight_stride < 0) return -1;
   if (heads == 1 && vdim >= 512 && vdim % 4 == 0 && vdim <= DS_THREADS * 16 && tokens < (1ll << 31) && gate_stride % 4 == 0 &&
       (((uintptr_t)x | (uintptr_t)weight | (uintptr_t)gate) & 15) == 0) {
 #define GW(T, PER) hipLaunchKernelGGL((wide_norm_gate_rows_kernel<T, PER>), dim3((unsigned)tokens), dim3(DS_THREADS), 0, stream,  \
                                       (T*)out, (const float*)x, (const float*)weight, (const float*)gate, gate_stride, vdim, eps, \
-                                      sigmoid_gate)
+                                      sigmoid_gate, out_stride, weight_stride, out_scale)
 #define GT(T) do { if (vdim <= DS_THREADS * 4) GW(T, 1); else if (vdim <= DS_THREADS * 8) GW(T, 2); else GW(T, 4); } while (0)
     if (out_bf16) GT(bf16_t); else GT(float);
 #undef GT
@@ -348,10 +351,12 @@ extern "C" int ga_head_norm_gate(void* out, const void* x, const void* weight, c
   if (heads == 1 && vdim >= 512 && tokens < (1ll << 31)) {          // a row of a wavefront's 64 lanes would be a long walk
     if (out_bf16)
       hipLaunchKernelGGL(wide_norm_gate_kernel<bf16_t>, dim3((unsigned)tokens), dim3(DS_THREADS), 0, stream, (bf16_t*)out,
-                         (const float*)x, (const float*)weight, (const float*)gate, gate_stride, vdim, eps, sigmoid_gate);
+                         (const float*)x, (const float*)weight, (const float*)gate, gate_stride, vdim, eps, sigmoid_gate, out_stride,
+                         weight_stride, out_scale);
     else
       hipLaunchKernelGGL(wide_norm_gate_kernel<float>, dim3((unsigned)tokens), dim3(DS_THREADS), 0, stream, (float*)out,
-                         (const float*)x, (const float*)weight, (const float*)gate, gate_stride, vdim, eps, sigmoid_gate);
+                         (const float*)x, (const float*)weight, (const float*)gate, gate_stride, vdim, eps, sigmoid_gate, out_stride,
+                         weight_stride, out_scale);
     return GA_CHECK_LAUNCH();
   }
   const int64_t rows = tokens * heads;
@@ -359,9 +364,11 @@ extern "C" int ga_head_norm_gate(void* out, const void* x, const void* weight, c
   dim3 grid((unsigned)((rows + per - 1) / per)), block(DS_THREADS);
   if (out_bf16)
     hipLaunchKernelGGL(head_norm_gate_kernel<bf16_t>, grid, block, 0, stream, (bf16_t*)out, (const float*)x,
-                       (const float*)weight, (const float*)gate, gate_stride, rows, heads, vdim, eps, sigmoid_gate);
+                       (const float*)weight, (const float*)gate, gate_stride, rows, heads, vdim, eps, sigmoid_gate, out_stride,
+                         weight_stride, out_scale);
   else
     hipLaunchKernelGGL(head_norm_gate_kernel<float>, grid, block, 0, stream, (float*)out, (const float*)x,
-                       (const float*)weight, (const float*)gate, gate_stride, rows, heads, vdim, eps, sigmoid_gate);
+                       (const float*)weight, (const float*)gate, gate_stride, rows, heads, vdim, eps, sigmoid_gate, out_stride,
+                         weight_stride, out_scale);
   return GA_CHECK_LAUNCH();
 }

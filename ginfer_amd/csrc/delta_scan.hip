@@ -1,0 +1,436 @@
+// Recurrences with a 32-bit state per request whose decay is one number per token and head: the gated delta rule and the
+// state-space recurrence of Mamba-2.  Per head, S is [dim, vdim] (its group's q and k, its own v):
+//   delta        S <- a S;  u = b (v - S^T k);  S <- S + k u^T;  o = S^T q          b = sigmoid(zb), q and k unit vectors
+//   state space  S <- a S + k (b v)^T;          o = S^T q + D v                     b = softplus(zb + bias)
+//   both         a = exp(-rate * softplus(za + bias))
+// q, k and v are columns of one 32-bit projection that have passed a short causal convolution over time (per channel) and silu;
+// za, zb and the gate z of the output are columns of the same projection.
+//   prepare   a step's convolved channels [tokens, channels] (float): a thread a channel and 8 tokens, unit vectors made in LDS
+//   scan      any entries: a workgroup owns (entry, head, 16 value columns) and walks the entry's tokens 16 at a time, their q,
+//             k and v in LDS, asked for a tile ahead.  16 lanes of a wavefront share a column: lane s keeps rows 64 j + 4 s .. + 3
+//             of it in registers, and their sums meet in four rotations inside the 16 lanes
+//   step      single tokens, all in one launch: a workgroup owns (entry, head), makes its channels, moves the state (all of
+//             its loads under way before the channels are made) and, for the delta rule, norms and gates the head's result
+// The sums of a token are taken in the same order in scan and step, so results do not depend on how the tokens were cut.
+// State layouts.  S: [slot][head][vdim / 4][dim / 64][lane][4], the order in which a wavefront reads it (rows beyond dim hold
+// zeros).  The convolution's inputs: a ring [slot][taps][channels], the row p % taps being position p's: a step's own row is
+// none of the taps - 1 rows it reads, so a workgroup may write it while another one still reads.
+#include "common.h"
+#include "ginfer_amd.h"
+
+#define DL_THREADS 256
+#define DL_WAVES (DL_THREADS / WAVE)
+#define DL_TILE 16           // tokens per trip through LDS
+#define DL_COLS 16           // value columns of a workgroup of the scan: four to a wavefront
+#define DL_MAX_TAPS 16
+#define DL_MAX_VDIM 512
+#define DL_PREP_TOKENS 8
+
+__device__ __forceinline__ float dl_silu(float z) { return z / (1.f + expf(-z)); }
+__device__ __forceinline__ float dl_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+
+// the sum over the 16 lanes of a row, the same bits in every lane: rotations by 8, 4, 2 and 1
+template <int CTRL>
+__device__ __forceinline__ float dl_rotated(float v) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xf, 0xf, false));
+}
+__device__ __forceinline__ float dl_row_sum(float v) {
+  v += dl_rotated<0x128>(v);
+  v += dl_rotated<0x124>(v);
+  v += dl_rotated<0x122>(v);
+  v += dl_rotated<0x121>(v);
+  return v;
+}
+
+// The input of channel c at `back` tokens before the token at row t (place `local` of its entry's tokens, position pos)
+__device__ __forceinline__ float dl_input(const ga_delta_args& a, int64_t t, int local, int pos, int64_t slot, int back, int c) {
+  if (local >= back) return a.proj[(t - back) * a.stride + a.conv_at + c];
+  if (pos < back) return 0.f;
+  return a.ring[(slot * a.taps + (pos - back) % a.taps) * (int64_t)a.channels + c];
+}
+
+// decay and step of a head at row t
+__device__ __forceinline__ float2 dl_coefficients(const ga_delta_args& a, int64_t t, int h) {
+  const float* row = a.proj + t * a.stride;
+  const float sp = dl_softplus(row[a.a_at + h] + a.dt_bias[h]);
+  const float decay = expf(-a.rate[h] * sp);
+  return make_float2(decay, a.delta ? 1.f / (1.f + expf(-row[a.b_at + h])) : sp);
+}
+
+// 1 / the length of x[0 .. n) (n elements in LDS), by one wavefront
+__device__ __forceinline__ float dl_inverse_length(const float* x, int n, float eps, int lane) {
+  float ss = 0.f;
+  for (int i = lane; i < n; i += WAVE) ss = fmaf(x[i], x[i], ss);
+  return 1.f / sqrtf(wave_sum(ss) + eps);
+}
+
+// A token's share of one column in a lane: rows 64 j + 4 s .. + 3
+template <int R4, bool DELTA>
+__device__ __forceinline__ float dl_advance(float4 (&S)[R4], const float4 (&k)[R4], const float4 (&q)[R4], float v, float a, float b) {
+  float u;
+  if (DELTA) {
+    float d0 = 0.f, d1 = 0.f;
+#pragma unroll
+    for (int j = 0; j < R4; ++j) {
+      d0 = fmaf(S[j].x, k[j].x, d0);
+      d1 = fmaf(S[j].y, k[j].y, d1);
+      d0 = fmaf(S[j].z, k[j].z, d0);
+      d1 = fmaf(S[j].w, k[j].w, d1);
+    }
+    u = b * (v - a * dl_row_sum(d0 + d1));
+  } else {
+    u = b * v;
+  }
+  float o0 = 0.f, o1 = 0.f;
+#pragma unroll
+  for (int j = 0; j < R4; ++j) {
+    S[j].x = fmaf(k[j].x, u, a * S[j].x);
+    S[j].y = fmaf(k[j].y, u, a * S[j].y);
+    S[j].z = fmaf(k[j].z, u, a * S[j].z);
+    S[j].w = fmaf(k[j].w, u, a * S[j].w);
+    o0 = fmaf(S[j].x, q[j].x, o0);
+    o1 = fmaf(S[j].y, q[j].y, o1);
+    o0 = fmaf(S[j].z, q[j].z, o0);
+    o1 = fmaf(S[j].w, q[j].w, o1);
+  }
+  return dl_row_sum(o0 + o1);
+}
+
+// ---------------------------------------------------------------------------------------------------- prepare
+// grid (token tiles, channel blocks): first the blocks of whole q and k heads (DL_THREADS / dim heads each), then the others
+template <int TAPS, int TB>      // TAPS 0: any number
+__global__ __launch_bounds__(DL_THREADS) void delta_prepare_kernel(float* __restrict__ out, const ga_delta_args a,
+                                                                   const int32_t* __restrict__ token_entry, int tokens) {
+  __shared__ float ys[TB][DL_THREADS];
+  __shared__ float factor[TB][DL_THREADS];
+  const int tid = threadIdx.x;
+  const int unit_channels = a.delta ? 2 * a.groups * a.dim : 0;
+  const int heads_here = a.delta ? DL_THREADS / a.dim : 1, block_channels = heads_here * a.dim;
+  const int unit_blocks = a.delta ? (2 * a.groups + heads_here - 1) / heads_here : 0;
+  const bool unit = (int)blockIdx.y < unit_blocks;
+  int c, last;
+  if (unit) {
+    c = blockIdx.y * block_channels + tid;
+    last = min(unit_channels, (int)(blockIdx.y + 1) * block_channels);
+  } else {
+    c = unit_channels + (blockIdx.y - unit_blocks) * DL_THREADS + tid;
+    last = a.channels;
+  }
+  const bool live = c < last;
+  const int64_t t0 = (int64_t)blockIdx.x * TB;
+  const int nt = min((int64_t)TB, tokens - t0);
+  float y[TB];
+#pragma unroll
+  for (int i = 0; i < TB; ++i) y[i] = 0.f;
+  if (live) {
+    const int taps = TAPS ? TAPS : a.taps;
+    const float bias = a.conv_bias ? a.conv_bias[c] : 0.f;
+    const float* w = a.conv_w + (int64_t)c * taps;
+    if (TAPS) {
+      float wr[TAPS ? TAPS : 1], x[TB + (TAPS ? TAPS : 1)];      // x[TAPS - 1 + i]: the input of token t0 + i
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) wr[j] = w[j];
+      const float* col = a.proj + a.conv_at + c;
+#pragma unroll
+      for (int i = 1 - TAPS; i < TB; ++i) {
+        const int64_t t = t0 + i;
+        x[TAPS - 1 + i] = (t >= 0 && i < nt) ? col[t * a.stride] : 0.f;
+      }
+#pragma unroll
+      for (int i = 0; i < TB; ++i) {
+        if (i >= nt) break;
+        const int64_t t = t0 + i;
+        const int e = token_entry[t], local = (int)(t - a.cu[e]);
+        float acc = bias;
+        if (local >= TAPS - 1) {
+#pragma unroll
+          for (int j = 0; j < TAPS; ++j) acc = fmaf(wr[j], x[i + j], acc);
+        } else {
+          const int pos = a.q_start[e] + local;
+          const int64_t slot = a.slots[e];
+#pragma unroll
+          for (int j = 0; j < TAPS; ++j)
+            acc = fmaf(wr[j], local >= TAPS - 1 - j ? x[i + j] : dl_input(a, t, local, pos, slot, TAPS - 1 - j, c), acc);
+        }
+        y[i] = dl_silu(acc);
+      }
+    } else {
+      for (int i = 0; i < nt; ++i) {
+        const int64_t t = t0 + i;
+        const int e = token_entry[t], local = (int)(t - a.cu[e]), pos = a.q_start[e] + local;
+        const int64_t slot = taps > 1 ? a.slots[e] : 0;
+        float acc = bias;
+        for (int j = 0; j < taps; ++j) acc = fmaf(w[j], dl_input(a, t, local, pos, slot, taps - 1 - j, c), acc);
+        y[i] = dl_silu(acc);
+      }
+    }
+  }
+  if (!unit) {
+    if (live) {
+#pragma unroll
+      for (int i = 0; i < TB; ++i)
+        if (i < nt) out[(t0 + i) * a.channels + c] = y[i];
+    }
+    return;
+  }
+#pragma unroll
+  for (int i = 0; i < TB; ++i) ys[i][tid] = y[i];
+  __syncthreads();
+  for (int r = tid / WAVE; r < nt * heads_here; r += DL_WAVES) {
+    const int i = r / heads_here, hh = r % heads_here;
+    const float f = dl_inverse_length(&ys[i][hh * a.dim], a.dim, a.unit_eps, tid % WAVE);
+    if (tid % WAVE == 0) factor[i][hh] = f;
+  }
+  __syncthreads();
+  if (live) {
+    const float scale = c < a.groups * a.dim ? a.q_scale : 1.f;
+    const int hh = tid / a.dim;
+#pragma unroll
+    for (int i = 0; i < TB; ++i)
+      if (i < nt) out[(t0 + i) * a.channels + c] = y[i] * factor[i][hh] * scale;
+  }
+}
+
+// ---------------------------------------------------------------------------------------------------- scan
+// grid (entries, heads, blocks of 16 value columns).  act: the prepared channels [tokens, channels].  out float [tokens, heads,
+// vdim]: o, or for the state space (o + D v) silu(z).
+template <int R4, bool DELTA>
+__global__ __launch_bounds__(DL_THREADS) void delta_scan_kernel(float* __restrict__ out, const float* __restrict__ act,
+                                                                const ga_delta_args a) {
+  constexpr int DP = 64 * R4;
+  __shared__ __attribute__((aligned(16))) float ks[DL_TILE][DP], qs[DL_TILE][DP];
+  __shared__ float vs[DL_TILE][DL_COLS], os[DL_TILE][DL_COLS];
+  __shared__ float2 cf[DL_TILE];
+  const int e = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * DL_COLS;
+  const int first = a.cu[e], n = a.cu[e + 1] - first;
+  if (n <= 0) return;
+  const int tid = threadIdx.x, lane = tid % WAVE, wave = tid / WAVE, s = lane & 15, col = wave * 4 + (lane >> 4);
+  const int g = h / (a.heads / a.groups);
+  const int start = a.q_start[e];
+  const int64_t slot = a.slots[e];
+  const int blocks = (a.vdim + 3) / 4, cb = blockIdx.z * (DL_COLS / 4) + wave;
+  float4* st = reinterpret_cast<float4*>(a.state) + ((slot * a.heads + h) * blocks + cb) * (int64_t)(R4 * WAVE) + lane;
+  float4 S[R4];
+#pragma unroll
+  for (int j = 0; j < R4; ++j) S[j] = (start > 0 && cb < blocks) ? st[j * WAVE] : make_float4(0.f, 0.f, 0.f, 0.f);
+  constexpr int PER = DL_TILE * DP / DL_THREADS;
+  float rq[PER], rk[PER], rv, rz = 0.f;
+  float2 rc = make_float2(0.f, 0.f);
+  const float* qp = act + a.q_at + g * a.dim;
+  const float* kp = act + a.k_at + g * a.dim;
+  const float* vp = act + a.v_at + h * a.vdim + v0;
+  const int ft = tid / DL_COLS, fc = tid % DL_COLS;        // this thread's place in a tile of values and results
+  const bool col_ok = v0 + fc < a.vdim;
+  auto fetch = [&](int t0) {
+    const int nt = min(DL_TILE, n - t0);
+#pragma unroll
+    for (int x = 0; x < PER; ++x) {
+      const int idx = tid + x * DL_THREADS, tt = idx / DP, i = idx % DP;
+      const bool in = tt < nt && i < a.dim;
+      const int64_t at = (int64_t)(first + t0 + tt) * a.channels + i;
+      rq[x] = in ? qp[at] : 0.f;
+      rk[x] = in ? kp[at] : 0.f;
+    }
+    const bool in = ft < nt && col_ok;
+    rv = in ? vp[(int64_t)(first + t0 + ft) * a.channels + fc] : 0.f;
+    if (!DELTA) rz = in ? a.proj[(int64_t)(first + t0 + ft) * a.stride + a.gate_at + h * a.vdim + v0 + fc] : 0.f;
+    if (tid < nt) rc = dl_coefficients(a, first + t0 + tid, h);
+  };
+  const float skip = DELTA ? 0.f : a.skip[h];
+  fetch(0);
+  for (int t0 = 0; t0 < n; t0 += DL_TILE) {
+    const int nt = min(DL_TILE, n - t0);
+    __syncthreads();                                       // the tile before is read out
+#pragma unroll
+    for (int x = 0; x < PER; ++x) {
+      const int idx = tid + x * DL_THREADS;
+      qs[idx / DP][idx % DP] = rq[x];
+      ks[idx / DP][idx % DP] = rk[x];
+    }
+    vs[ft][fc] = rv;
+    if (tid < DL_TILE) cf[tid] = rc;
+    const float z = rz, v_own = rv;
+    __syncthreads();
+    if (t0 + DL_TILE < n) fetch(t0 + DL_TILE);
+#pragma unroll 4
+    for (int tt = 0; tt < nt; ++tt) {
+      float4 k[R4], q[R4];
+#pragma unroll
+      for (int j = 0; j < R4; ++j) {
+        k[j] = *reinterpret_cast<const float4*>(&ks[tt][64 * j + 4 * s]);
+        q[j] = *reinterpret_cast<const float4*>(&qs[tt][64 * j + 4 * s]);
+      }
+      const float o = dl_advance<R4, DELTA>(S, k, q, vs[tt][col], cf[tt].x, cf[tt].y);
+      if (s == 0) os[tt][col] = o;
+    }
+    __syncthreads();
+    if (ft < nt && col_ok) {
+      float o = os[ft][fc];
+      if (!DELTA) o = (o + skip * v_own) * dl_silu(z);
+      out[((int64_t)(first + t0 + ft) * a.heads + h) * a.vdim + v0 + fc] = o;
+    }
+  }
+  if (cb < blocks) {
+#pragma unroll
+    for (int j = 0; j < R4; ++j) st[j * WAVE] = S[j];
+  }
+  // the last taps inputs of the entry into the ring, the channels dealt to the entry's workgroups
+  if (a.taps > 1) {
+    const int per = gridDim.y * gridDim.z * DL_THREADS, mine = (h * gridDim.z + blockIdx.z) * DL_THREADS + tid;
+    for (int c = mine; c < a.channels; c += per)
+      for (int i = max(0, n - a.taps); i < n; ++i)
+        a.ring[(slot * a.taps + (start + i) % a.taps) * (int64_t)a.channels + c] = a.proj[(int64_t)(first + i) * a.stride + a.conv_at + c];
+  }
+}
+
+// ---------------------------------------------------------------------------------------------------- step
+// grid (entries, heads): every entry brings one token.  DELTA: out T [tokens, ..] (row stride out_stride), the head's columns
+// from h * vdim on, out_scale * weight * silu(gate) * o / rms(o); else float, (o + D v) silu(gate).
+template <int R4, bool DELTA, typename T>
+__global__ __launch_bounds__(DL_THREADS) void delta_step_kernel(T* __restrict__ out, int64_t out_stride, const ga_delta_args a,
+                                                                const float* __restrict__ weight, float eps, float out_scale) {
+  constexpr int NB = 16 / R4;                              // column blocks that a wavefront has in registers at a time
+  __shared__ __attribute__((aligned(16))) float ks[64 * R4], qs[64 * R4];
+  __shared__ float vs[DL_MAX_VDIM], os[DL_MAX_VDIM];
+  __shared__ float scratch[DL_WAVES], lengths[2];
+  const int e = blockIdx.x, h = blockIdx.y;
+  const int64_t t = a.cu[e];
+  if (a.cu[e + 1] - (int)t <= 0) return;
+  const int tid = threadIdx.x, lane = tid % WAVE, wave = tid / WAVE, s = lane & 15;
+  const int per_group = a.heads / a.groups, g = h / per_group;
+  const int pos = a.q_start[e];
+  const int64_t slot = a.slots[e];
+  const int blocks = (a.vdim + 3) / 4;
+  float4* st = reinterpret_cast<float4*>(a.state) + (slot * a.heads + h) * blocks * (int64_t)(R4 * WAVE) + lane;
+  float4 S[NB][R4];
+  auto load = [&](int first) {
+#pragma unroll
+    for (int b = 0; b < NB; ++b) {
+      const int cb = first + b * DL_WAVES + wave;
+#pragma unroll
+      for (int j = 0; j < R4; ++j)
+        S[b][j] = (pos > 0 && cb < blocks) ? st[(int64_t)cb * (R4 * WAVE) + j * WAVE] : make_float4(0.f, 0.f, 0.f, 0.f);
+    }
+  };
+  load(0);
+  const float2 c2 = dl_coefficients(a, t, h);
+  for (int i = tid; i < 64 * R4; i += DL_THREADS)
+    if (i >= a.dim) ks[i] = qs[i] = 0.f;
+  // the convolved channels: this head's values, its group's q and k
+  for (int i = tid; i < 2 * a.dim + a.vdim; i += DL_THREADS) {
+    const int c = i < a.dim ? a.q_at + g * a.dim + i : i < 2 * a.dim ? a.k_at + g * a.dim + (i - a.dim) : a.v_at + h * a.vdim + (i - 2 * a.dim);
+    const float own = a.proj[t * a.stride + a.conv_at + c];
+    const float* w = a.conv_w + (int64_t)c * a.taps;
+    float acc = a.conv_bias ? a.conv_bias[c] : 0.f;
+    for (int j = 0; j < a.taps - 1; ++j) acc = fmaf(w[j], dl_input(a, t, 0, pos, slot, a.taps - 1 - j, c), acc);
+    const float y = dl_silu(fmaf(w[a.taps - 1], own, acc));
+    if (a.taps > 1 && (i >= 2 * a.dim || h == g * per_group)) a.ring[(slot * a.taps + pos % a.taps) * (int64_t)a.channels + c] = own;
+    if (i < a.dim) qs[i] = y;
+    else if (i < 2 * a.dim) ks[i - a.dim] = y;
+    else vs[i - 2 * a.dim] = y;
+  }
+  __syncthreads();
+  if (DELTA) {
+    if (wave < 2) {
+      const float f = dl_inverse_length(wave ? ks : qs, a.dim, a.unit_eps, lane);
+      if (lane == 0) lengths[wave] = f;
+    }
+    __syncthreads();
+  }
+  float4 k[R4], q[R4];
+  const float fq = DELTA ? lengths[0] : 1.f, fk = DELTA ? lengths[1] : 1.f, sq = DELTA ? a.q_scale : 1.f;
+#pragma unroll
+  for (int j = 0; j < R4; ++j) {
+    k[j] = *reinterpret_cast<const float4*>(&ks[64 * j + 4 * s]);
+    q[j] = *reinterpret_cast<const float4*>(&qs[64 * j + 4 * s]);
+    if (DELTA) {
+      k[j].x *= fk; k[j].y *= fk; k[j].z *= fk; k[j].w *= fk;
+      q[j].x = q[j].x * fq * sq; q[j].y = q[j].y * fq * sq; q[j].z = q[j].z * fq * sq; q[j].w = q[j].w * fq * sq;
+    }
+  }
+  for (int first = 0; first < blocks; first += NB * DL_WAVES) {
+    if (first > 0) load(first);
+#pragma unroll
+    for (int b = 0; b < NB; ++b) {
+      const int cb = first + b * DL_WAVES + wave;
+      if (cb < blocks) {
+        const int col = cb * 4 + (lane >> 4);
+        const float o = dl_advance<R4, DELTA>(S[b], k, q, col < a.vdim ? vs[col] : 0.f, c2.x, c2.y);
+#pragma unroll
+        for (int j = 0; j < R4; ++j) st[(int64_t)cb * (R4 * WAVE) + j * WAVE] = S[b][j];
+        if (s == 0 && col < a.vdim) os[col] = o;
+      }
+    }
+  }
+  __syncthreads();
+  const float* gate = a.proj + t * a.stride + a.gate_at + h * a.vdim;
+  T* op = out + t * out_stride + (int64_t)h * a.vdim;
+  if (DELTA) {
+    float ss = 0.f;
+    for (int i = tid; i < a.vdim; i += DL_THREADS) ss = fmaf(os[i], os[i], ss);
+    ss = block_sum<DL_WAVES>(ss, scratch);
+    const float rms = sqrtf(ss / (float)a.vdim + eps);
+    for (int i = tid; i < a.vdim; i += DL_THREADS) Num<T>::st(op + i, os[i] / rms * weight[i] * dl_silu(gate[i]) * out_scale);
+  } else {
+    const float skip = a.skip[h];
+    for (int i = tid; i < a.vdim; i += DL_THREADS) Num<T>::st(op + i, (os[i] + skip * vs[i]) * dl_silu(gate[i]));
+  }
+}
+
+static int dl_check(const ga_delta_args& a) {
+  if (a.heads <= 0 || a.groups <= 0 || a.heads % a.groups || a.dim <= 0 || a.dim > 256 || a.vdim <= 0 || a.vdim > DL_MAX_VDIM) return -1;
+  if (a.taps < 1 || a.taps > DL_MAX_TAPS || (a.taps > 1 && !a.ring) || !a.conv_w) return -2;
+  if (a.heads > 65535) return -3;
+  if (!a.proj || !a.state || !a.slots || !a.cu || !a.q_start || !a.rate || !a.dt_bias || (!a.delta && !a.skip)) return -4;
+  return 0;
+}
+
+extern "C" int ga_delta_prepare(void* act, const ga_delta_args* args, const void* token_entry, int tokens, hipStream_t stream) {
+  if (tokens <= 0) return 0;
+  const ga_delta_args& a = *args;
+  const int rc = dl_check(a);
+  if (rc) return rc;
+  const int units = a.delta ? 2 * a.groups : 0, heads_here = a.delta ? DL_THREADS / a.dim : 1;
+  const int plain = a.channels - units * a.dim;
+  const int64_t blocks = (units + heads_here - 1) / heads_here + (plain + DL_THREADS - 1) / DL_THREADS;
+  if (plain < 0 || blocks > 65535) return -5;
+#define GO(TAPS, TB) hipLaunchKernelGGL((delta_prepare_kernel<TAPS, TB>), dim3((tokens + TB - 1) / TB, (unsigned)blocks), dim3(DL_THREADS), 0, \
+                                        stream, (float*)act, a, (const int32_t*)token_entry, tokens)
+  const bool few = (int64_t)tokens * blocks <= 2048;         // a token to a workgroup while that does not fill the chip
+  if (a.taps == 4) { if (few) GO(4, 1); else GO(4, DL_PREP_TOKENS); }
+  else { if (few) GO(0, 1); else GO(0, DL_PREP_TOKENS); }
+#undef GO
+  return GA_CHECK_LAUNCH();
+}
+
+extern "C" int ga_delta_scan(void* out, const void* act, const ga_delta_args* args, int entries, hipStream_t stream) {
+  if (entries <= 0) return 0;
+  const ga_delta_args& a = *args;
+  const int rc = dl_check(a);
+  if (rc) return rc;
+  dim3 grid(entries, a.heads, (a.vdim + DL_COLS - 1) / DL_COLS), block(DL_THREADS);
+#define GO(R4, D) hipLaunchKernelGGL((delta_scan_kernel<R4, D>), grid, block, 0, stream, (float*)out, (const float*)act, a)
+#define GR(D) do { const int r = (a.dim + 63) / 64; if (r == 1) GO(1, D); else if (r == 2) GO(2, D); else if (r == 3) GO(3, D); else GO(4, D); } while (0)
+  if (a.delta) GR(true); else GR(false);
+#undef GR
+#undef GO
+  return GA_CHECK_LAUNCH();
+}
+
+extern "C" int ga_delta_step(void* out, int64_t out_stride, const ga_delta_args* args, const void* weight, float eps, float out_scale,
+                             int out_bf16, int entries, hipStream_t stream) {
+  if (entries <= 0) return 0;
+  const ga_delta_args& a = *args;
+  const int rc = dl_check(a);
+  if (rc) return rc;
+  if (a.delta ? !weight : out_bf16) return -6;
+  dim3 grid(entries, a.heads), block(DL_THREADS);
+#define GO(R4, D, T) hipLaunchKernelGGL((delta_step_kernel<R4, D, T>), grid, block, 0, stream, (T*)out, out_stride, a, (const float*)weight, eps, out_scale)
+#define GR(D, T) do { const int r = (a.dim + 63) / 64; if (r == 1) GO(1, D, T); else if (r == 2) GO(2, D, T); else if (r == 3) GO(3, D, T); else GO(4, D, T); } while (0)
+  if (!a.delta) GR(false, float);
+  else if (out_bf16) GR(true, bf16_t);
+  else GR(true, float);
+#undef GR
+#undef GO
+  return GA_CHECK_LAUNCH();
+}

@@ -6,7 +6,8 @@
 //   gate-up  act[r, c] = silu(w g) * (w u) (weight_inside) or w * silu(g) * u, g = x[token of r] . Wg_e[c], u = ... Wu_e[c],
 //            w the pair's weight; r is the place in the grouped order
 //   down     parts[k][t][:] = Wd_e act[r], r the place of pair t * top + k: every choice's result by itself, in 32-bit, for the
-//            consumer to add in the order of the choice
+//            consumer to add in the order of the choice.  Choices that name no expert here (experts without weights) are left out of
+//            everything
 // Weights lie as the dense product over all experts has them: expert e's ff gate rows and then its ff up rows in one matrix
 // [experts * 2 ff, hidden], the down matrices side by side in one [hidden, experts * ff].
 //
@@ -117,10 +118,10 @@ extern "C" int ga_expert_plan(const void* ids, void* pair_of_row, void* tiles, v
 
 // The plan of a step of up to 64 pairs, worked out by every wavefront for itself (lane p holds pair p): experts in the order of
 // their first pair.  false: there is no tile of this number.  Writes the tile's pairs (every wavefront the same ones).
-__device__ __forceinline__ bool es_plan_tile(const int32_t* __restrict__ ids, int pairs, int tile, int tile_rows, int& e, int& r0,
-                                             int& rows, int32_t* tile_pairs, int lane) {
+__device__ __forceinline__ bool es_plan_tile(const int32_t* __restrict__ ids, int pairs, int experts, int tile, int tile_rows, int& e,
+                                             int& r0, int& rows, int32_t* tile_pairs, int lane) {
   const int id = lane < pairs ? ids[lane] : -1;
-  uint64_t left = __ballot(lane < pairs);
+  uint64_t left = __ballot(id >= 0 && id < experts);         // choices beyond the experts that have weights are not ours
   int first = 0;
   while (left) {
     e = __builtin_amdgcn_readlane(id, __builtin_ctzll(left));
@@ -146,8 +147,8 @@ __global__ __launch_bounds__(KW * WAVE) void expert_few_kernel(void* __restrict_
                                                                const bf16_t* __restrict__ w, int64_t w_expert, int64_t w_row,
                                                                const float* __restrict__ weights, const int32_t* __restrict__ pair_of_row,
                                                                const int32_t* __restrict__ tiles, const int32_t* __restrict__ count,
-                                                               const int32_t* __restrict__ ids, int K, int cols, int top, int tokens,
-                                                               int inside) {
+                                                               const int32_t* __restrict__ ids, int experts, int K, int cols, int top,
+                                                               int tokens, int inside) {
   constexpr int MM = MATS * MB;                              // operands of the weights: block mb of matrix m at m * MB + mb
   __shared__ float red[KW][MM * NT][4][WAVE];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c = lane & 15, g = lane >> 4;
@@ -160,7 +161,7 @@ __global__ __launch_bounds__(KW * WAVE) void expert_few_kernel(void* __restrict_
     r0 = tiles[4 * tile + 1];
     rows = tiles[4 * tile + 2];
     for (int i = threadIdx.x; i < rows; i += KW * WAVE) tile_pairs[i] = pair_of_row[r0 + i];
-  } else if (!es_plan_tile(ids, top * tokens, blockIdx.y, 16 * NT, e, r0, rows, tile_pairs, lane)) {
+  } else if (!es_plan_tile(ids, top * tokens, experts, blockIdx.y, 16 * NT, e, r0, rows, tile_pairs, lane)) {
     return;                                                  // the whole workgroup: every wavefront comes to the same tile
   }
   __syncthreads();
@@ -366,8 +367,8 @@ __global__ __launch_bounds__(128 * WN, (WN == 1 ? 1 : 2)) void expert_many_kerne
 // -64; needs K in steps of 32).  Operands bfloat16 at 16-byte addresses, K and cols multiples of 8.
 template <int MATS>
 static int eg_launch(void* out, const void* in, const void* w, int64_t w_expert, int64_t w_row, const void* weights,
-                     const void* pair_of_row, const void* tiles, const void* count, const void* ids, int max_tiles, int K, int cols,
-                     int top, int tokens, int inside, int tile_rows, hipStream_t stream) {
+                     const void* pair_of_row, const void* tiles, const void* count, const void* ids, int experts, int max_tiles, int K,
+                     int cols, int top, int tokens, int inside, int tile_rows, hipStream_t stream) {
   if (tokens <= 0 || max_tiles <= 0) return 0;
   if (K <= 0 || K % 8 || cols <= 0 || cols % 8 || top <= 0 || w_row % 8 || w_expert % 8 ||
       (((uintptr_t)out | (uintptr_t)in | (uintptr_t)w) & 15))
@@ -379,7 +380,7 @@ static int eg_launch(void* out, const void* in, const void* w, int64_t w_expert,
 #define SIZES K, cols, top, tokens, inside
 #define FEW(NT, MB, KW)                                                                                                       \
   hipLaunchKernelGGL((expert_few_kernel<MATS, NT, MB, KW>), dim3((cols + 16 * MB - 1) / (16 * MB), max_tiles), dim3(KW * WAVE), \
-                     0, stream, OPERANDS, (const int32_t*)ids, SIZES)
+                     0, stream, OPERANDS, (const int32_t*)ids, experts, SIZES)
 #define MANY(WN)                                                                                                              \
   do {                                                                                                                        \
     const int64_t n = (int64_t)((cols + 256 / MATS - 1) / (256 / MATS)) * max_tiles;                                          \
@@ -406,15 +407,15 @@ static int eg_launch(void* out, const void* in, const void* w, int64_t w_expert,
 }
 
 extern "C" int ga_expert_gate_up(void* act, const void* x, const void* w_gate_up, const void* weights, const void* pair_of_row,
-                                 const void* tiles, const void* count, const void* ids, int max_tiles, int hidden, int ff, int top,
+                                 const void* tiles, const void* count, const void* ids, int experts, int max_tiles, int hidden, int ff, int top,
                                  int tokens, int weight_inside, int tile_rows, hipStream_t stream) {
-  return eg_launch<2>(act, x, w_gate_up, (int64_t)2 * ff * hidden, hidden, weights, pair_of_row, tiles, count, ids, max_tiles, hidden, ff,
+  return eg_launch<2>(act, x, w_gate_up, (int64_t)2 * ff * hidden, hidden, weights, pair_of_row, tiles, count, ids, experts, max_tiles, hidden, ff,
                       top, tokens, weight_inside, tile_rows, stream);
 }
 
 extern "C" int ga_expert_down(void* parts, const void* act, const void* w_down, int64_t w_row, const void* pair_of_row,
-                              const void* tiles, const void* count, const void* ids, int max_tiles, int hidden, int ff, int top,
+                              const void* tiles, const void* count, const void* ids, int experts, int max_tiles, int hidden, int ff, int top,
                               int tokens, int tile_rows, hipStream_t stream) {
-  return eg_launch<1>(parts, act, w_down, ff, w_row, nullptr, pair_of_row, tiles, count, ids, max_tiles, ff, hidden, top, tokens, 0,
+  return eg_launch<1>(parts, act, w_down, ff, w_row, nullptr, pair_of_row, tiles, count, ids, experts, max_tiles, ff, hidden, top, tokens, 0,
                       tile_rows, stream);
 }

@@ -93,11 +93,11 @@ int ga_scalar_rmsnorm_rows(void* out, const void* x, const void* gain, const voi
 int ga_add_scalar_rmsnorm(void* residual, const void* y, const void* gain, void* copy, int tokens, int hidden, float eps,
                           int y_bf16, int gain_bf16, hipStream_t stream);
 
-// ---- embedding_sinusoid.hip: out float [tokens, hidden] = table[ids] + (sin | cos)(position * freq[i / 2]), then the norm
+// ---- embedding_sinusoid.hip: out float [tokens, hidden] = table_scale * table[ids] + (sin | cos)(position * freq[i / 2]), then the norm
 // with one gain (gain null: no norm); freq float [(hidden + 1) / 2]
 int ga_embedding_sinusoid_norm(void* out, const void* table, const void* ids, const void* positions, const void* freq,
                                const void* gain, int tokens, int hidden, float eps, int table_bf16, int gain_bf16,
-                               hipStream_t stream);
+                               float table_scale, hipStream_t stream);
 
 // ---- short_conv.hip: causal convolution of `taps` taps over time on each channel of the float stream x [tokens, width],
 // w float [width, taps]; the inputs before a step's tokens come from state float [slots, taps - 1, width].  apply: out
@@ -170,23 +170,28 @@ int ga_latent_output_few(void* o, const void* a, const void* w_uv, const void* g
 // tokens_per_workgroup neighbouring tokens share a workgroup's tiles of keys and values (0: the library chooses; -1: the
 // same, and every request of the step has at least 8 tokens in it); few_tokens_workgroups, fill_workgroups: the two
 // thresholds by which the launcher chooses among its kernels (speed only); sink_scores: null, or one float per head: a
-// score that every query of the head sees beside its keys' and that has no value (it only enters the denominator)
+// score that every query of the head sees beside its keys' and that has no value (it only enters the denominator); cap: 0, or
+// scores become cap * tanh(score / cap); gate: null, or float rows of a number per head (row stride gate_stride) whose
+// sigmoid, times gate_scale, multiplies the head's result
 int ga_paged_attention_generic(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* k_pages,
                                const void* v_pages, const void* block_table, int table_width, const void* token_entry,
                                const void* positions, int tokens, int nh, int nkv, int hd, int page_size, int window,
                                float scale, int is_bf16, int tokens_per_workgroup, int few_tokens_workgroups,
-                               int fill_workgroups, const void* sink_scores, hipStream_t stream);
+                               int fill_workgroups, const void* sink_scores, float cap, const void* gate, int64_t gate_stride,
+                               float gate_scale, hipStream_t stream);
 
 // ---- attention_mfma.hip (one library per head size): bfloat16 on the matrix cores
 int ga_attn_head_dim();
 int ga_attn_prefill_max_tile_rows();
-// sinks (both entry points): null, or one float per head, a score that enters every denominator of the head
+// sinks (both entry points): null, or one float per head, a score that enters every denominator of the head; cap (0 unless
+// the library was built with SOFT_CAP=1, then positive) and gate as for the general kernels
 // single new tokens; workspace_o: n_tokens * nh * num_splits * head_dim floats, workspace_ml: n_tokens * nh *
 // num_splits * 2 floats
 int ga_attn_decode(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* k_pages,
                    const void* v_pages, const void* block_table, int table_width, const void* decode_info, int n_tokens,
                    int nh, int nkv, int page_size, int window, float scale, int split_keys, int num_splits,
-                   void* workspace_o, void* workspace_ml, const void* sinks, hipStream_t stream);
+                   void* workspace_o, void* workspace_ml, const void* sinks, float cap, const void* gate, int64_t gate_stride,
+                   float gate_scale, hipStream_t stream);
 // rows of prompt portions, in tiles of int32 x 4 = (entry, first row of the step, rows, first position).  parts (or
 // null): per tile int32 x 4 = (first key, end of keys, index of the tile's first row among the rows that come in parts,
 // part + (number of parts << 16)): the keys of such a tile are dealt to several workgroups, whose partial results
@@ -196,7 +201,7 @@ int ga_attn_prefill(void* out, int64_t out_stride, const void* q, int64_t q_stri
                     const void* v_pages, const void* block_table, int table_width, const void* tiles, int n_tiles,
                     int tile_rows, int nh, int nkv, int page_size, int window, float scale, int fill_workgroups,
                     int prefer_workgroups, const void* parts, const void* part_rows, int n_part_rows, int num_parts, void* part_o,
-                    void* part_ml, const void* sinks, hipStream_t stream);
+                    void* part_ml, const void* sinks, float cap, const void* gate, int64_t gate_stride, float gate_scale, hipStream_t stream);
 
 // ---- conv_rope_kv.hip: behind a fused q|k|v projection proj [tokens, (nh + nkv) hd + nkv vd] whose channels pass a
 // causal convolution of `taps` taps over time (w float [channels, taps], or null with taps 1: none; state float [slots,
@@ -204,12 +209,13 @@ int ga_attn_prefill(void* out, int64_t out_stride, const void* q, int64_t q_stri
 // q's and k's heads (cos_t, sin_t float [positions, rotary_dim / 2], or null with rotary_dim 0), q into q_out [tokens, nh
 // * padded], k and v into their pages (k [pages, nkv, page_size, padded], v [pages, nkv, padded, page_size]), heads
 // padded with zeros; then (update_state) a second launch moves the state on by the step's tokens; proj may be float
-// beside a bfloat16 compute dtype (proj_bf16 0, is_bf16 1)
+// beside a bfloat16 compute dtype (proj_bf16 0, is_bf16 1); stride: proj's row stride; head_eps >= 0: every head of q and k is
+// divided by its own root mean square and multiplied by gain float [2, hd] (q's, then k's)
 int ga_conv_rope_kv(void* q_out, const void* proj, const void* w, void* state, const void* slots, const void* token_entry,
                     const void* cu, const void* q_start, const void* positions, const void* cos_t, const void* sin_t,
                     const void* slot_mapping, void* k_pages, void* v_pages, int tokens, int entries, int nh, int nkv, int hd,
                     int vd, int padded, int rotary_dim, int taps, int page_size, int write_kv, int update_state, int is_bf16,
-                    int proj_bf16, void* row_scale, const void* gain, float norm_eps, hipStream_t stream);
+                    int proj_bf16, void* row_scale, const void* gain, float norm_eps, int64_t stride, float head_eps, hipStream_t stream);
 
 // ---- output_norm.hip: residual[t] += scale * gain * y[t] / sqrt(mean(y[t]^2) + eps) (a norm on a sublayer's output, a
 // factor per channel behind it; gain and scale float [hidden], scale may be null); with `next` also next[t] = next_gain *
@@ -226,11 +232,15 @@ int ga_output_norm_add(void* residual, const void* y, const void* gain, const vo
 // width], column c weighted by dense[t, c / ff] (columns behind experts * ff by 1)
 int ga_route_topk(void* ids, void* weights, void* dense, const void* scores, int tokens, int experts, int top,
                   hipStream_t stream);
-// the same outputs from sigmoid scores: choice by s + correction inside the `keep` best of `groups` groups (a group's score:
-// its group_top largest choice scores added), weights s (/ (their sum + floor) where normalise) * scale
-int ga_route_sigmoid_groups(void* ids, void* weights, void* dense, const void* logits, const void* correction, int tokens,
-                            int experts, int top, int groups, int keep, int group_top, int normalise, float floor, float scale,
-                            hipStream_t stream);
+// the same outputs from a score of every expert (softmax: the softmax over all of them; else the sigmoid): choice by s +
+// correction (float [experts] or null) inside the `keep` best of `groups` groups (a group's score:
+// its group_top largest choice scores added), weights s (/ (their sum + floor) where normalise) * scale.
+// The last `identity` experts have no weights: their result is x itself (the token's row, in the compute dtype), written times
+// the weight to own_out: float [top][tokens][hidden] at those choices (by_choice), or float [tokens][hidden] summed; dense has
+// rows of the other experts only
+int ga_route_groups(void* ids, void* weights, void* dense, const void* logits, const void* correction, int tokens, int experts,
+                    int top, int groups, int keep, int group_top, int normalise, float floor, float scale, int softmax,
+                    int identity, const void* x, int x_bf16, int hidden, void* own_out, int by_choice, hipStream_t stream);
 // weight_inside: silu(w gate) * (w up), the weight multiplying what the expert reads
 int ga_weighted_silu_mul(void* out, const void* gate_up, const void* dense, int tokens, int width, int experts, int ff,
                          int weight_inside, int is_bf16, hipStream_t stream);
@@ -257,10 +267,10 @@ int ga_combine_pairs(void* out, const void* y, const void* shared, const void* w
 int ga_expert_plan(const void* ids, void* pair_of_row, void* tiles, void* count, int pairs, int experts, int tile_rows,
                    int max_tiles, hipStream_t stream);
 int ga_expert_gate_up(void* act, const void* x, const void* w_gate_up, const void* weights, const void* pair_of_row,
-                      const void* tiles, const void* count, const void* ids, int max_tiles, int hidden, int ff, int top,
+                      const void* tiles, const void* count, const void* ids, int experts, int max_tiles, int hidden, int ff, int top,
                       int tokens, int weight_inside, int tile_rows, hipStream_t stream);
 int ga_expert_down(void* parts, const void* act, const void* w_down, int64_t w_row, const void* pair_of_row, const void* tiles,
-                   const void* count, const void* ids, int max_tiles, int hidden, int ff, int top, int tokens, int tile_rows, hipStream_t stream);
+                   const void* count, const void* ids, int experts, int max_tiles, int hidden, int ff, int top, int tokens, int tile_rows, hipStream_t stream);
 
 // ---- activation.hip: out[i] = max(x[i], 0)^2 over `total` elements (out may be x)
 int ga_relu_square(void* out, const void* x, int64_t total, int is_bf16, hipStream_t stream);
@@ -296,9 +306,44 @@ int ga_gla_decay(void* decay, const void* low, int64_t low_stride, const void* a
                  int channels, int rank, float tau, hipStream_t stream);
 // out [tokens, heads, vdim] = x / rms(x over vdim) (* weight [vdim], or null) (* silu(gate), or sigmoid(gate) where sigmoid_gate;
 // 32-bit rows with a stride, or null); heads == 1 with a wide vdim: a norm over all heads together
+// (weight_stride vdim: every head has a weight of its own; the result times out_scale, rows out_stride apart)
 // (decay_scan's silu_inputs: the recurrence reads silu(q), silu(k), silu(v))
 int ga_head_norm_gate(void* out, const void* x, const void* weight, const void* gate, int64_t gate_stride, int64_t tokens,
-                      int heads, int vdim, float eps, int out_bf16, int sigmoid_gate, hipStream_t stream);
+                      int heads, int vdim, float eps, int out_bf16, int sigmoid_gate, int64_t out_stride, int weight_stride,
+                      float out_scale, hipStream_t stream);
+
+// ---- delta_scan.hip: recurrences with one decay per token and head over float state: the gated delta rule (delta 1) and the
+// state-space recurrence of Mamba-2 (delta 0); the equations stand in the source.  proj: 32-bit rows; conv_at: its first
+// convolved channel, q_at, k_at, v_at: where q [groups dim], k [groups dim] and v [heads vdim] lie among the convolved channels
+// (delta: q | k | v in this order from 0 on); a_at, b_at, gate_at: columns of the decay's and the step's numbers per head and
+// of the output's gate [heads vdim]; conv_w float [channels, taps], conv_bias float [channels] or null; rate, dt_bias, skip
+// float [heads] (skip: delta 0 only); ring float [slots, taps, channels] (null for one tap), state float [slots, heads,
+// (vdim + 3) / 4, (dim + 63) / 64, 256]
+typedef struct {
+  const float* proj;
+  int64_t stride;
+  const float* conv_w;
+  const float* conv_bias;
+  const float* rate;
+  const float* dt_bias;
+  const float* skip;
+  float* ring;
+  float* state;
+  const int64_t* slots;
+  const int32_t* cu;
+  const int32_t* q_start;
+  int conv_at, q_at, k_at, v_at, a_at, b_at, gate_at;
+  int channels, taps, heads, groups, dim, vdim, delta;
+  float q_scale, unit_eps;
+} ga_delta_args;
+// act float [tokens, channels]: convolved, silu, q and k (delta) as unit vectors, q times q_scale
+int ga_delta_prepare(void* act, const ga_delta_args* args, const void* token_entry, int tokens, hipStream_t stream);
+// out float [tokens, heads, vdim]: o (delta), or (o + skip v) silu(gate); advances state and ring
+int ga_delta_scan(void* out, const void* act, const ga_delta_args* args, int entries, hipStream_t stream);
+// every entry brings one token: all of it in one launch; delta: out (compute dtype, row stride out_stride) = out_scale * weight *
+// silu(gate) * o / rms(o), else float, as the scan's
+int ga_delta_step(void* out, int64_t out_stride, const ga_delta_args* args, const void* weight, float eps, float out_scale,
+                  int out_bf16, int entries, hipStream_t stream);
 
 // ---- pooled_attention.hip: attention over a window of tokens and the means of the blocks before it, sigmoid weights.
 // prepare: q and k of a 32-bit projection [q heads | k heads | v heads ...] turned by position (pairs 2i, 2i + 1), divided by

@@ -70,30 +70,50 @@ __global__ __launch_bounds__(ROUTE_THREADS) void route_topk_kernel(const float* 
   }
 }
 
-// Routing by sigmoid scores with a correction and groups of experts (one wavefront per token):
-//   s = sigmoid(z);  c = s + correction (the choice score; without a correction c = s)
+// Routing by scores of every expert with a correction and groups of experts (one wavefront per token):
+//   s = sigmoid(z), or (softmax) the softmax of z over all experts;  c = s + correction (the choice score; without a correction c = s)
 //   the experts fall into `groups` equal groups of neighbours; a group's score is the sum of its `group_top` largest c; only
 //   the experts of the `keep` best groups can be chosen (groups == 1: all of them)
 //   the `top` experts with the largest c among those are chosen (the lowest index among equals)
 //   weights: the chosen experts' s, divided by their sum + floor where `normalise`, times `scale`
-// Written as route_topk_kernel writes them: ids and weights [T, top], and a row of weights over all experts.
+// Written as route_topk_kernel writes them: ids and weights [T, top], and a row of weights over the first `own` experts.
+// The experts from `own` on are identity experts: their result is the token's row itself (x, in the compute dtype, hidden
+// wide), times the weight.  own_out, where there are any: float, by choice [top][T][hidden] (the places of the choices that are
+// identity experts are written, the others left), or summed [T][hidden] (by_choice 0: every row is written).
 #define ROUTE_GROUP_TOP_MAX 4
-__global__ __launch_bounds__(ROUTE_THREADS) void route_sigmoid_groups_kernel(
+template <typename T>
+__global__ __launch_bounds__(ROUTE_THREADS) void route_groups_kernel(
     const float* __restrict__ logits, const float* __restrict__ correction, int32_t* __restrict__ ids,
     float* __restrict__ weights, float* __restrict__ dense, int experts, int top, int groups, int keep, int group_top,
-    int normalise, float floor, float scale) {
+    int normalise, float floor, float scale, int softmax, int own, const T* __restrict__ x, int hidden,
+    float* __restrict__ own_out, int by_choice) {
   constexpr int PER = ROUTE_MAX_EXPERTS / ROUTE_THREADS;
   __shared__ float choice[ROUTE_MAX_EXPERTS], plain[ROUTE_MAX_EXPERTS], group_score[ROUTE_MAX_EXPERTS];
   __shared__ int32_t kept[ROUTE_MAX_EXPERTS], chosen_i[ROUTE_MAX_EXPERTS];
   const int64_t t = blockIdx.x;
   const int lane = threadIdx.x;
-  float c[PER];
+  float c[PER], zs[PER];
   bool taken[PER];
+  float most = -INFINITY, total_exp = 0.f;
 #pragma unroll
   for (int j = 0; j < PER; ++j) {
     const int e = lane + j * ROUTE_THREADS;
-    float z = e < experts ? logits[t * experts + e] : 0.f;
-    float s = 1.0f / (1.0f + expf(-z));
+    zs[j] = e < experts ? logits[t * experts + e] : -INFINITY;
+    most = fmaxf(most, zs[j]);
+  }
+  if (softmax) {
+    most = wave_max(most);
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      zs[j] = expf(zs[j] - most);
+      total_exp += zs[j];
+    }
+    total_exp = wave_sum(total_exp);
+  }
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    const int e = lane + j * ROUTE_THREADS;
+    float s = softmax ? zs[j] / total_exp : 1.0f / (1.0f + expf(-zs[j]));
     c[j] = e < experts ? s + (correction ? correction[e] : 0.f) : -INFINITY;
     // what is no number (the rows that pad a recorded step may hold anything) counts as the smallest
     if (!(c[j] == c[j])) { c[j] = -INFINITY; s = 0.f; }
@@ -160,13 +180,29 @@ __global__ __launch_bounds__(ROUTE_THREADS) void route_sigmoid_groups_kernel(
   float total = 0.f;
   for (int k = 0; k < top; ++k) total += plain[chosen_i[k]];             // in the order of the choice
   const float factor = normalise ? scale / (total + floor) : scale;
-  for (int e = lane; e < experts; e += ROUTE_THREADS) dense[t * experts + e] = 0.f;
+  for (int e = lane; e < own; e += ROUTE_THREADS) dense[t * own + e] = 0.f;
   __syncthreads();
   for (int k = lane; k < top; k += ROUTE_THREADS) {
     const float w = plain[chosen_i[k]] * factor;
     ids[t * top + k] = chosen_i[k];
     weights[t * top + k] = w;
-    dense[t * experts + chosen_i[k]] = w;
+    if (chosen_i[k] < own) dense[t * own + chosen_i[k]] = w;
+  }
+  if (own_out == nullptr) return;
+  const T* row = x + t * hidden;
+  if (by_choice) {
+    for (int k = 0; k < top; ++k) {
+      if (chosen_i[k] < own) continue;
+      const float w = plain[chosen_i[k]] * factor;
+      float* o = own_out + ((int64_t)k * gridDim.x + t) * hidden;
+      for (int i = lane; i < hidden; i += ROUTE_THREADS) o[i] = w * Num<T>::ld(row + i);
+    }
+  } else {
+    float w = 0.f;
+    for (int k = 0; k < top; ++k)
+      if (chosen_i[k] >= own) w += plain[chosen_i[k]] * factor;
+    float* o = own_out + t * hidden;
+    for (int i = lane; i < hidden; i += ROUTE_THREADS) o[i] = w == 0.f ? 0.f : w * Num<T>::ld(row + i);
   }
 }
 
@@ -349,16 +385,21 @@ extern "C" int ga_route_topk(void* ids, void* weights, void* dense, const void* 
   return GA_CHECK_LAUNCH();
 }
 
-extern "C" int ga_route_sigmoid_groups(void* ids, void* weights, void* dense, const void* logits, const void* correction,
-                                       int tokens, int experts, int top, int groups, int keep, int group_top, int normalise,
-                                       float floor, float scale, hipStream_t stream) {
+extern "C" int ga_route_groups(void* ids, void* weights, void* dense, const void* logits, const void* correction, int tokens,
+                               int experts, int top, int groups, int keep, int group_top, int normalise, float floor, float scale,
+                               int softmax, int identity, const void* x, int x_bf16, int hidden, void* own_out, int by_choice,
+                               hipStream_t stream) {
   if (tokens <= 0) return 0;
   if (experts <= 0 || experts > ROUTE_MAX_EXPERTS || top <= 0 || top > experts) return -1;
   if (groups < 1 || experts % groups || keep < 1 || keep > groups || top > keep * (experts / groups)) return -2;
   if (group_top < 1 || group_top > ROUTE_GROUP_TOP_MAX) return -3;
-  hipLaunchKernelGGL(route_sigmoid_groups_kernel, dim3(tokens), dim3(ROUTE_THREADS), 0, stream, (const float*)logits,
-                     (const float*)correction, (int32_t*)ids, (float*)weights, (float*)dense, experts, top, groups, keep,
-                     group_top, normalise, floor, scale);
+  if (identity < 0 || identity >= experts || (identity > 0 && (!x || !own_out || hidden <= 0))) return -4;
+#define GO(T) hipLaunchKernelGGL(route_groups_kernel<T>, dim3(tokens), dim3(ROUTE_THREADS), 0, stream, (const float*)logits,      \
+                                 (const float*)correction, (int32_t*)ids, (float*)weights, (float*)dense, experts, top, groups, keep, \
+                                 group_top, normalise, floor, scale, softmax, experts - identity, (const T*)x, hidden,            \
+                                 identity > 0 ? (float*)own_out : nullptr, by_choice)
+  if (x_bf16) GO(bf16_t); else GO(float);
+#undef GO
   return GA_CHECK_LAUNCH();
 }
 

@@ -26,7 +26,7 @@ FLAGS = ["--offload-arch=" + ARCH, "-O3", "-std=c++17", "-shared", "-fPIC",
 MODULES = ("embedding", "norm", "rope_kv", "attention_generic", "attention_mfma", "gemm", "gemm_skinny",
            "activation", "sampling", "random_fill", "scalar_norm", "embedding_sinusoid", "short_conv", "gated_recurrence",
            "latent_attention", "output_norm", "routing", "conv_rope_kv", "decay_scan", "pooled_attention",
-           "gated_residual", "hyper_connection", "rglru", "layer_norm", "expert_gemm")
+           "gated_residual", "hyper_connection", "rglru", "layer_norm", "expert_gemm", "delta_scan")
 # flags of single modules: the random-weights generator must round every operation by itself, as the host's twin does
 MODULE_FLAGS = {"random_fill": ["-ffp-contract=off"], "attention_generic": ["-ffp-contract=off"]}
 # headers beside common.h that a module includes (they enter its digest)
@@ -37,7 +37,8 @@ HOST_FLAGS = ["-O2", "-std=c++17", "-shared", "-fPIC", "-pthread", "-ffp-contrac
 HOST_HEADERS = {"random_fill_host": ["random_normal.h"]}
 # Modules that are compiled for one value of a parameter (a macro) at a time; build_all() without a
 # list compiles these values, and any other value a model needs is compiled when it is first asked for.
-VARIANTS = {"attention_mfma": [{"HEAD_DIM": hd} for hd in range(16, 257, 16)]}
+VARIANTS = {"attention_mfma": [{"HEAD_DIM": hd} for hd in range(16, 257, 16)]
+            + [{"HEAD_DIM": hd, "SOFT_CAP": 1} for hd in range(16, 257, 16)]}
 
 _loaded = {}
 _lock = threading.Lock()

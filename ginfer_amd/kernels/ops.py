@@ -257,8 +257,25 @@ def _check_sinks(sinks, num_heads, device):
     return sinks
 
 
+def _head_extras(soft_cap, gate, gate_scale, tokens, num_heads):
+    """The launchers' arguments for capped scores and gated heads: soft_cap None, or the bound of scores that become soft_cap *
+    tanh(score / soft_cap); gate None, or float32 rows [T, heads] (unit inner stride) whose sigmoid, times gate_scale,
+    multiplies the heads' results."""
+    cap = 0.0 if soft_cap is None else float(soft_cap)
+    _need(soft_cap is None or cap > 0.0, "scores are capped by a positive number, got %r", soft_cap)
+    stride = 0
+    if gate is not None:
+        _dev(gate)
+        _need(gate.dtype == torch.float32 and tuple(gate.shape) == (tokens, num_heads) and (num_heads == 1 or gate.stride(1) == 1),
+              "the heads' gate must be float32 [%d, %d] with unit inner stride, got %s %s", tokens, num_heads, gate.dtype,
+              tuple(gate.shape))
+        stride = gate.stride(0)
+    return _f(cap), _ptr(gate), _i64(stride), _f(gate_scale)
+
+
 def paged_attention_generic(q, k_pages, v_pages, block_table, token_entry, positions, num_heads, num_kv_heads,
-                            head_dim, scale, window=None, out=None, tokens_per_workgroup=0, sinks=None):
+                            head_dim, scale, window=None, out=None, tokens_per_workgroup=0, sinks=None, soft_cap=None, gate=None,
+                            gate_scale=1.0):
     """q: rows of the fused projection ([T, >= nh*hd]; the first nh*hd columns are the queries).
     Token t attends to the keys of request token_entry[t] at positions
     [max(0, p - window + 1), p], p = positions[t] (window may be any value of `mask_parameter`: negative for chunks).  Returns [T, nh*hd].  tokens_per_workgroup: how many neighbouring
@@ -281,7 +298,7 @@ def paged_attention_generic(q, k_pages, v_pages, block_table, token_entry, posit
         _i(block_table.shape[1]), _ptr(token_entry), _ptr(positions), _i(T), _i(num_heads), _i(num_kv_heads),
         _i(head_dim), _i(k_pages.shape[2]), _i(int(window) if window else 0), _f(scale), _i(_is_bf16(q.dtype)),
         _i(int(tokens_per_workgroup)), _i(TUNING.generic_few_tokens_workgroups), _i(TUNING.generic_fill_workgroups),
-        _ptr(sinks), _stream()), "paged_attention_generic")
+        _ptr(sinks), *_head_extras(soft_cap, gate, gate_scale, T, num_heads), _stream()), "paged_attention_generic")
     return out
 
 
@@ -563,6 +580,11 @@ def first_visible_key(pos, mask):
     return 0
 
 
+def attention_mfma_module(head_dim, capped=False):
+    """The library of the matrix-core attention for this head size, for plain or for capped scores: (source, macros)."""
+    return ("attention_mfma", dict({"HEAD_DIM": head_dim}, **({"SOFT_CAP": 1} if capped else {})))
+
+
 def attention_mfma_supported(dtype, head_dim, page_size):
     return (dtype == torch.bfloat16 and head_dim in MFMA_HEAD_DIMS and page_size >= 8
             and page_size & (page_size - 1) == 0)
@@ -690,7 +712,7 @@ def _decode_splits(plan, window, nkv, head_blocks):
 
 
 def paged_attention_mfma(q, k_pages, v_pages, block_table, step, num_heads, num_kv_heads, head_dim, scale,
-                         window=None, out=None, sinks=None):
+                         window=None, out=None, sinks=None, soft_cap=None, gate=None, gate_scale=1.0):
     """bfloat16 attention of every token of the step on the matrix cores: single new tokens through the
     split-key kernel, rows of prompt portions through the tiled kernel."""
     T = _check_attention_operands(q, k_pages, v_pages, block_table, step.token_entry, step.positions, num_heads,
@@ -706,7 +728,8 @@ def paged_attention_mfma(q, k_pages, v_pages, block_table, step, num_heads, num_
           "the matrix-core attention kernels count the rows of a layer's cache in 32 bits: %d pages x %d kv heads x "
           "%d is too many",
           k_pages.shape[0], num_kv_heads, max(page_size, head_dim))
-    lib = build.load("attention_mfma", {"HEAD_DIM": head_dim})
+    extras = _head_extras(soft_cap, gate, gate_scale, T, num_heads)
+    lib = build.load(*attention_mfma_module(head_dim, soft_cap is not None))
     _need(lib.ga_attn_head_dim() == head_dim, "attention library was built for another head size")
     # rows of a prompt portion per wavefront: 32 where the kernel has it and the step is long, else 16
     wide = T >= TUNING.prefill_wide_tiles_from
@@ -717,7 +740,8 @@ def paged_attention_mfma(q, k_pages, v_pages, block_table, step, num_heads, num_
     _need(sum(step.host_q_len) == T, "the step's entries do not add up to its tokens")
     if out is None:
         out = torch.empty((T, num_heads * head_dim), dtype=q.dtype, device=q.device)
-    _need(out.dtype == q.dtype and out.shape == (T, num_heads * head_dim) and out.is_contiguous(), "out must be [T, nh*hd]")
+    _need(out.dtype == q.dtype and out.shape == (T, num_heads * head_dim) and out.stride(1) == 1 and out.stride(0) % 4 == 0
+          and out.data_ptr() % 8 == 0, "out must be [T, nh*hd] with rows at 8-byte addresses")
     w = int(window) if window else 0
     if plan["n_decode"]:
         group = num_heads // num_kv_heads
@@ -728,7 +752,7 @@ def paged_attention_mfma(q, k_pages, v_pages, block_table, step, num_heads, num_
         _check(lib.ga_attn_decode(
             _ptr(out), _i64(out.stride(0)), _ptr(q), _i64(q.stride(0)), _ptr(k_pages), _ptr(v_pages), _ptr(block_table),
             _i(block_table.shape[1]), _ptr(plan["decode_info"]), _i(plan["n_decode"]), _i(num_heads), _i(num_kv_heads), _i(page_size), _i(w), _f(scale), _i(split_keys),
-            _i(num_splits), _ptr(ws_o), _ptr(ws_ml), _ptr(sinks), _stream()), "attn_decode")
+            _i(num_splits), _ptr(ws_o), _ptr(ws_ml), _ptr(sinks), *extras, _stream()), "attn_decode")
     if plan["n_tiles"]:
         part_o = part_ml = None
         if plan["n_part_rows"]:
@@ -740,7 +764,7 @@ def paged_attention_mfma(q, k_pages, v_pages, block_table, step, num_heads, num_
             _i(block_table.shape[1]), _ptr(plan["tiles"]), _i(plan["n_tiles"]), _i(tile_rows), _i(num_heads), _i(num_kv_heads),
             _i(page_size), _i(w), _f(scale), _i(TUNING.prefill_fill_workgroups), _i(TUNING.prefill_prefer_workgroups),
             _ptr(plan["parts"]), _ptr(plan["part_rows"]),
-            _i(plan["n_part_rows"]), _i(plan["num_parts"]), _ptr(part_o), _ptr(part_ml), _ptr(sinks), _stream()), "attn_prefill")
+            _i(plan["n_part_rows"]), _i(plan["num_parts"]), _ptr(part_o), _ptr(part_ml), _ptr(sinks), *extras, _stream()), "attn_prefill")
     return out
 
 
@@ -774,16 +798,18 @@ def _prefill_workgroups(step, tile_rows, group, nkv, head_dim, window):
 
 
 def paged_attention(q, k_pages, v_pages, block_table, step, num_heads, num_kv_heads, head_dim, scale, window=None,
-                    sinks=None, chunk=None):
+                    sinks=None, chunk=None, soft_cap=None, gate=None, gate_scale=1.0, out=None):
     """Attention of every token of the step over its request's pages.  window: the last `window` keys; chunk: the keys of
     the query's own chunk of `chunk` positions, counted from position 0 (neither: every earlier key).  Chooses the kernel: the general
     one in 32-bit (fixed order of every sum: bit-identical however the work is cut); in bfloat16 the
     matrix-core kernels where they take the shape.  sinks: None, or float32 [num_heads], a score per head that
-    enters every denominator of the softmax and has no value."""
+    enters every denominator of the softmax and has no value.  soft_cap: scores become soft_cap * tanh(score / soft_cap).  gate:
+    float32 [T, num_heads] rows; head h's result is multiplied by gate_scale * sigmoid(gate[:, h]).  out: where the result
+    goes, [T, num_heads * head_dim] with unit inner stride (columns of a wider tensor, say)."""
     window = mask_parameter(window, chunk) or None
     if attention_mfma_supported(q.dtype, head_dim, k_pages.shape[2]):
         return paged_attention_mfma(q, k_pages, v_pages, block_table, step, num_heads, num_kv_heads, head_dim, scale,
-                                    window, sinks=sinks)
+                                    window, sinks=sinks, soft_cap=soft_cap, gate=gate, gate_scale=gate_scale, out=out)
     if step.max_q_len == 1:
         grouping = 1
     elif "static_plan" not in (step.extra or {}) and min(step.host_q_len) >= 8:
@@ -791,7 +817,8 @@ def paged_attention(q, k_pages, v_pages, block_table, step, num_heads, num_kv_he
     else:
         grouping = 0
     return paged_attention_generic(q, k_pages, v_pages, block_table, step.token_entry, step.positions, num_heads,
-                                   num_kv_heads, head_dim, scale, window, tokens_per_workgroup=grouping, sinks=sinks)
+                                   num_kv_heads, head_dim, scale, window, tokens_per_workgroup=grouping, sinks=sinks,
+                                   soft_cap=soft_cap, gate=gate, gate_scale=gate_scale, out=out)
 
 
 # ---------------------------------------------------------------------------------------------------------------------
@@ -856,8 +883,9 @@ def add_scalar_rmsnorm(residual, y, gain, eps, copy=False):
     return out if out is not None else residual
 
 
-def embedding_sinusoid_norm(table, ids, positions, freq, gain, eps):
-    """table [V, H], ids and positions int32 [T], freq float32 [(H + 1) // 2], gain: one number or None -> float32 [T, H]."""
+def embedding_sinusoid_norm(table, ids, positions, freq, gain, eps, table_scale=1.0):
+    """table [V, H], ids and positions int32 [T], freq float32 [(H + 1) // 2], gain: one number or None (no norm) -> float32
+    [T, H]: table_scale * the table's rows + the positions' sines and cosines, normed."""
     _dev(table, ids, positions, freq, gain)
     _need(table.dim() == 2 and table.is_contiguous(), "embedding table must be contiguous [V, H]")
     T, H = ids.shape[0], table.shape[1]
@@ -868,7 +896,7 @@ def embedding_sinusoid_norm(table, ids, positions, freq, gain, eps):
     lib = build.load("embedding_sinusoid")
     _check(lib.ga_embedding_sinusoid_norm(_ptr(out), _ptr(table), _ptr(ids), _ptr(positions), _ptr(freq), _ptr(gain), _i(T),
                                           _i(H), _f(eps), _i(_is_bf16(table.dtype)),
-                                          _i(_scalar_gain(gain) if gain is not None else 0), _stream()), "embedding_sinusoid_norm")
+                                          _i(_scalar_gain(gain) if gain is not None else 0), _f(table_scale), _stream()), "embedding_sinusoid_norm")
     return out
 
 
@@ -1190,12 +1218,17 @@ def route_topk(scores, top):
     return ids, weights, dense
 
 
-def route_sigmoid_groups(logits, top, correction=None, groups=1, keep=1, group_top=2, normalise=True, floor=0.0, scale=1.0):
-    """logits float32 [T, E] -> (ids, weights, dense) as `route_topk` gives them, from sigmoid scores s = sigmoid(logits): the
-    choice goes by s + correction (float32 [E] or None); the experts fall into `groups` equal groups of neighbours, a group's
-    score is the sum of its `group_top` largest choice scores, and only experts of the `keep` best groups can be chosen; the
-    weights are the chosen experts' s, divided by their sum + floor where `normalise`, times scale."""
-    _dev(logits, correction)
+def route_groups(logits, top, correction=None, groups=1, keep=1, group_top=2, normalise=True, floor=0.0, scale=1.0, softmax=False,
+                 identity=0, x=None, own_out=None):
+    """logits float32 [T, E] -> (ids, weights, dense) as `route_topk` gives them, from a score of every expert, s =
+    sigmoid(logits) or (softmax) the softmax over all of them: the choice goes by s + correction (float32 [E] or None); the
+    experts fall into `groups` equal groups of neighbours, a group's score is the sum of its `group_top` largest choice scores,
+    and only experts of the `keep` best groups can be chosen; the weights are the chosen experts' s, divided by their sum + floor
+    where `normalise`, times scale.
+    The last `identity` experts give the token's row x [T, H] itself, times the weight, written to own_out: float32 [top, T, H]
+    at the choices that name one (the other places are left as they are), or float32 [T, H]: their sum (zeros where none is
+    chosen).  `dense` then has rows of E - identity weights."""
+    _dev(logits, correction, x, own_out)
     _need(logits.dtype == torch.float32 and logits.dim() == 2 and logits.is_contiguous(), "logits must be contiguous float32 [T, E]")
     T, E = logits.shape
     _need(1 <= E <= ROUTE_MAX_EXPERTS and 1 <= top <= E, "routing takes 1 to %d experts and 1 <= top <= experts; got %d, top %d",
@@ -1205,13 +1238,23 @@ def route_sigmoid_groups(logits, top, correction=None, groups=1, keep=1, group_t
           group_top, top)
     if correction is not None:
         _f32(correction, (E,), "correction")
+    _need(0 <= identity < E, "%d identity experts of %d", identity, E)
+    H, by_choice = 0, False
+    if identity:
+        _need(x is not None and x.dim() == 2 and x.shape[0] == T and x.is_contiguous() and x.dtype in (torch.float32, torch.bfloat16),
+              "identity experts need the tokens' rows, contiguous float32 or bfloat16 [%d, H]", T)
+        H = x.shape[1]
+        by_choice = own_out is not None and own_out.dim() == 3
+        _f32(own_out, (top, T, H) if by_choice else (T, H), "own_out")
     ids = torch.empty((T, top), dtype=torch.int32, device=logits.device)
     weights = torch.empty((T, top), dtype=torch.float32, device=logits.device)
-    dense = torch.empty((T, E), dtype=torch.float32, device=logits.device)
+    dense = torch.empty((T, E - identity), dtype=torch.float32, device=logits.device)
     lib = build.load("routing")
-    _check(lib.ga_route_sigmoid_groups(_ptr(ids), _ptr(weights), _ptr(dense), _ptr(logits), _ptr(correction), _i(T), _i(E), _i(top),
-                                       _i(groups), _i(keep), _i(group_top), _i(1 if normalise else 0), _f(floor), _f(scale),
-                                       _stream()), "route_sigmoid_groups")
+    _check(lib.ga_route_groups(_ptr(ids), _ptr(weights), _ptr(dense), _ptr(logits), _ptr(correction), _i(T), _i(E), _i(top),
+                               _i(groups), _i(keep), _i(group_top), _i(1 if normalise else 0), _f(floor), _f(scale),
+                               _i(1 if softmax else 0), _i(identity), _ptr(x if identity else None),
+                               _i(_is_bf16(x.dtype) if identity else 0), _i(H), _ptr(own_out if identity else None),
+                               _i(1 if by_choice else 0), _stream()), "route_groups")
     return ids, weights, dense
 
 
@@ -1311,12 +1354,13 @@ def expert_rows_supported(x, hidden, ff):
     return x.dtype == torch.bfloat16 and hidden % 8 == 0 and ff % 8 == 0 and x.is_contiguous() and x.data_ptr() % 16 == 0
 
 
-def experts_over_their_rows(x, ids, weights, w_gate_up, w_down, experts, ff, weight_inside, tile_rows):
+def experts_over_their_rows(x, ids, weights, w_gate_up, w_down, experts, ff, weight_inside, tile_rows, parts=None):
     """x bfloat16 [T, H]; ids int32 [T, top] and weights float32 [T, top] of the chosen experts; w_gate_up [experts * 2 ff (..), H]
     (an expert's gate rows, then its up rows) and w_down [H, experts * ff (..)] -> float32 [top, T, H]: result k of token t is
     Wdown_e (silu(w g) * (w u)) (weight_inside) or Wdown_e (w * silu(g) * u) of its k-th choice e.  Nothing waits for the host.
     tile_rows: rows of an expert that a workgroup takes at a time, 16, 32 or 64 (weights streamed from memory once for that
-    many), -64, 128 or 256 (64, 128 or 256 rows by tiles of the weights through LDS; H and ff in steps of 32)."""
+    many), -64, 128 or 256 (64, 128 or 256 rows by tiles of the weights through LDS; H and ff in steps of 32).  Choices that name no
+    expert below `experts` are left out: their places of `parts` (the result, where the caller brings it) stay as they are."""
     _dev(x, ids, weights, w_gate_up, w_down)
     T, H = x.shape
     top = ids.shape[1]
@@ -1339,16 +1383,18 @@ def experts_over_their_rows(x, ids, weights, w_gate_up, w_down, experts, ff, wei
         tiles, pair_of_row, count = plan[:4 * max_tiles], plan[4 * max_tiles:4 * max_tiles + P], plan[4 * max_tiles + P:]
     own = ids if inside else None
     act = torch.empty((P, ff), dtype=x.dtype, device=x.device)
-    parts = torch.empty((top, T, H), dtype=torch.float32, device=x.device)
+    if parts is None:
+        parts = torch.empty((top, T, H), dtype=torch.float32, device=x.device)
+    _f32(parts, (top, T, H), "parts")
     lib = build.load("expert_gemm")
     if not inside:
         _check(lib.ga_expert_plan(_ptr(ids), _ptr(pair_of_row), _ptr(tiles), _ptr(count), _i(P), _i(experts), _i(rows), _i(max_tiles),
                                   _stream()), "expert_plan")
     _check(lib.ga_expert_gate_up(_ptr(act), _ptr(x), _ptr(w_gate_up), _ptr(weights), _ptr(pair_of_row), _ptr(tiles), _ptr(count), _ptr(own),
-                                 _i(max_tiles), _i(H), _i(ff), _i(top), _i(T), _i(1 if weight_inside else 0), _i(tile_rows),
+                                 _i(experts), _i(max_tiles), _i(H), _i(ff), _i(top), _i(T), _i(1 if weight_inside else 0), _i(tile_rows),
                                  _stream()), "expert_gate_up")
     _check(lib.ga_expert_down(_ptr(parts), _ptr(act), _ptr(w_down), _i64(w_down.stride(0)), _ptr(pair_of_row), _ptr(tiles),
-                              _ptr(count), _ptr(own), _i(max_tiles), _i(H), _i(ff), _i(top), _i(T), _i(tile_rows), _stream()), "expert_down")
+                              _ptr(count), _ptr(own), _i(experts), _i(max_tiles), _i(H), _i(ff), _i(top), _i(T), _i(tile_rows), _stream()), "expert_down")
     return parts
 
 
@@ -1443,19 +1489,21 @@ def scaled_sum(a, b, sa, sb, dtype):
 
 
 def conv_rope_kv(proj, weight, state, slots, step, cos, sin, slot_mapping, k_pages, v_pages, num_heads, num_kv_heads, head_dim,
-                 value_dim, padded, dtype, write_kv=True, update_state=True, qk_gain=None, qk_eps=0.0):
+                 value_dim, padded, dtype, write_kv=True, update_state=True, qk_gain=None, qk_eps=0.0, head_norm=False):
     """Behind a fused q|k|v projection whose channels pass a short causal convolution: proj [T, (nh + nkv) hd + nkv vd] in
     the compute dtype `dtype` or in float32; weight float32 [channels, taps] (None: no convolution); state float32 [slots, taps - 1, channels]
     (None for one tap) and slots int64 [entries]; cos, sin float32 [positions, rotary_dim / 2] (None: no rotation).
     qk_gain float32 [(nh + nkv) hd] (no convolution then): q and k are divided by the root mean square of the token's WHOLE q
     (k) projection (eps qk_eps) and multiplied by the gain, before the rotation.
+    head_norm: qk_gain is float32 [2, hd] instead, and every head of q and of k is divided by its own root mean square and
+    multiplied by its kind's gain.  proj's rows may be longer than its C columns (a view of a wider tensor).
     Returns q [T, nh * padded], heads padded with zeros, and writes k and v (padded alike) into the pages at slot_mapping;
     moves the state on by the step's tokens."""
     _dev(proj, weight, state, slots, cos, sin, slot_mapping, k_pages, v_pages)
     T = proj.shape[0]
     C = (num_heads + num_kv_heads) * head_dim + num_kv_heads * value_dim
-    _need(proj.dim() == 2 and proj.shape[1] == C and proj.is_contiguous() and proj.dtype in (torch.float32, torch.bfloat16),
-          "proj must be contiguous float32 or bfloat16 [T, %d], got %s %s", C, proj.dtype, tuple(proj.shape))
+    _need(proj.dim() == 2 and proj.shape[1] == C and proj.stride(1) == 1 and proj.stride(0) >= C and proj.dtype in (torch.float32, torch.bfloat16),
+          "proj must be float32 or bfloat16 [T, %d] with unit inner stride, got %s %s", C, proj.dtype, tuple(proj.shape))
     _need(head_dim <= padded <= 256 and value_dim <= padded, "heads padded to %d (at most 256) do not hold %d / %d", padded,
           head_dim, value_dim)
     _need(num_heads + 2 * num_kv_heads <= 65535, "too many heads for one launch: %d", num_heads + 2 * num_kv_heads)
@@ -1487,7 +1535,10 @@ def conv_rope_kv(proj, weight, state, slots, step, cos, sin, slot_mapping, k_pag
     _need(proj.dtype in (dtype, torch.float32), "proj must be %s or float32", dtype)
     q = torch.empty((T, num_heads * padded), dtype=dtype, device=proj.device)
     row_scale = None
-    if qk_gain is not None:
+    if head_norm:
+        _f32(qk_gain, (2, head_dim), "qk_gain")
+        _need(qk_gain.device == proj.device and qk_eps >= 0.0, "qk_gain lies on another device, or its eps is negative")
+    elif qk_gain is not None:
         _need(weight is None, "the norm over the whole projection stands in front of no convolution")
         _f32(qk_gain, ((num_heads + num_kv_heads) * head_dim,), "qk_gain")
         _need(qk_gain.device == proj.device, "qk_gain lies on another device")
@@ -1498,8 +1549,8 @@ def conv_rope_kv(proj, weight, state, slots, step, cos, sin, slot_mapping, k_pag
                                _ptr(slot_mapping), _ptr(k_pages), _ptr(v_pages), _i(T), _i(E), _i(num_heads), _i(num_kv_heads),
                                _i(head_dim), _i(value_dim), _i(padded), _i(rotary_dim), _i(taps), _i(page_size),
                                _i(1 if write_kv else 0), _i(1 if update_state else 0), _i(_is_bf16(dtype)),
-                               _i(_is_bf16(proj.dtype)), _ptr(row_scale), _ptr(qk_gain), _f(qk_eps), _stream()),
-           "conv_rope_kv")
+                               _i(_is_bf16(proj.dtype)), _ptr(row_scale), _ptr(qk_gain), _f(qk_eps),
+                               _i64(proj.stride(0)), _f(qk_eps if head_norm else -1.0), _stream()), "conv_rope_kv")
     return q
 
 
@@ -1580,25 +1631,131 @@ def decay_scan(proj, q_start, k_start, v_start, state, slots, step, heads, dim, 
     return out
 
 
-def head_norm_gate(x, weight, eps, dtype, proj=None, gate_start=0, sigmoid_gate=False):
+def head_norm_gate(x, weight, eps, dtype, proj=None, gate_start=0, sigmoid_gate=False, out=None, out_scale=1.0):
     """x float32 [T, heads, V] -> [T, heads * V] in `dtype`: every head's row divided by its root mean square, times weight
-    [V] (None: no weight), times silu of the gate (its sigmoid where sigmoid_gate), the columns gate_start .. gate_start +
-    heads * V of the float32 projection `proj` (None: no gate).  A norm over all heads together is the case heads = 1."""
-    _dev(x, weight, proj)
+    ([V], shared by the heads, or [heads, V]; None: no weight), times silu of the gate (its sigmoid where sigmoid_gate), the
+    columns gate_start .. gate_start + heads * V of the float32 projection `proj` (None: no gate), times out_scale.  A norm
+    over all heads together is the case heads = 1.  out: where the result goes, rows with unit inner stride."""
+    _dev(x, weight, proj, out)
     _need(x.dtype == torch.float32 and x.dim() == 3 and x.is_contiguous(), "x must be contiguous float32 [T, heads, V]")
     T, H, V = x.shape
     if weight is not None:
-        _f32(weight, (V,), "weight")
+        _f32(weight, (V,) if weight.dim() == 1 else (H, V), "weight")
     gate = None
     if proj is not None:
         _need(proj.shape[0] == T, "the gate has %d rows, x has %d", proj.shape[0], T)
         gate = _rows_of(proj, gate_start, H * V, "gate")
-    out = torch.empty((T, H * V), dtype=dtype, device=x.device)
+    if out is None:
+        out = torch.empty((T, H * V), dtype=dtype, device=x.device)
+    _need(tuple(out.shape) == (T, H * V) and out.dtype == dtype and out.stride(1) == 1, "out must be %s [%d, %d] with unit inner stride",
+          dtype, T, H * V)
     lib = build.load("decay_scan")
     _check(lib.ga_head_norm_gate(_ptr(out), _ptr(x), _ptr(weight), _ptr(gate), _i64(proj.stride(0) if proj is not None else 0),
                                  _i64(T), _i(H), _i(V), _f(eps), _i(_is_bf16(dtype)), _i(1 if sigmoid_gate else 0),
+                                 _i64(out.stride(0)), _i(V if weight is not None and weight.dim() == 2 else 0), _f(out_scale),
                                  _stream()), "head_norm_gate")
     return out
+
+
+# ---------------------------------------------------------------------------------------------------------------------
+# recurrences with one decay per token and head: the gated delta rule, the state-space recurrence
+
+DELTA_MAX_DIM = 256
+DELTA_MAX_VDIM = 512
+
+
+class _DeltaArgs(ctypes.Structure):
+    """ga_delta_args (csrc/ginfer_amd.h)."""
+    _fields_ = ([("proj", _vp), ("stride", _i64)] + [(n, _vp) for n in ("conv_w", "conv_bias", "rate", "dt_bias", "skip", "ring", "state",
+                                                                        "slots", "cu", "q_start")]
+                + [(n, _i) for n in ("conv_at", "q_at", "k_at", "v_at", "a_at", "b_at", "gate_at", "channels", "taps", "heads", "groups",
+                                     "dim", "vdim", "delta")] + [("q_scale", _f), ("unit_eps", _f)])
+
+
+def delta_state_shape(heads, dim, vdim):
+    """The state of such a recurrence per request, as its kernels read it: float32 [heads, vdim / 4, dim / 64, 64 * 4]."""
+    return (heads, -(-vdim // 4), -(-dim // 64), 256)
+
+
+def delta_state_matrix(state, dim, vdim):
+    """[.., heads, dim, vdim] of a state in the kernels' layout: element [cb, j, lane, i] is row 64 j + 4 (lane % 16) + i of
+    column 4 cb + lane / 16."""
+    lead, (blocks, r4) = state.shape[:-3], state.shape[-3:-1]
+    s = state.reshape(lead + (blocks, r4, 4, 16, 4))             # cb, j, column, s, i
+    n = len(lead)
+    s = s.permute(tuple(range(n)) + (n + 1, n + 3, n + 4, n, n + 2)).reshape(lead + (r4 * 64, blocks * 4))
+    return s[..., :dim, :vdim]
+
+
+def delta_recurrence(proj, conv_weight, conv_bias, rate, dt_bias, skip, ring, state, slots, step, heads, groups, dim, vdim, columns, delta,
+                     q_scale=1.0, unit_eps=0.0, weight=None, eps=0.0, dtype=None, out=None, out_scale=1.0):
+    """One step of the recurrence (csrc/delta_scan.hip has the equations) over per-request state.  proj: float32 [T, ..] rows with
+    unit inner stride; `columns` names where its parts begin: conv (the convolved channels), a and b (the decay's and the
+    step's numbers per head), gate [heads * vdim], and, among the convolved channels, q, k and v.  conv_weight float32 [channels,
+    taps], conv_bias float32 [channels] or None; rate, dt_bias float32 [heads]; ring float32 [slots, taps, channels] (None for
+    one tap) and state float32 [slots, *delta_state_shape] are advanced in place.
+    delta: returns [T, heads * vdim] in `dtype`: out_scale * weight * silu(gate) * o / rms(o) per head (weight float32 [vdim]),
+    into `out` where it is given.  Else: float32 [T, heads, vdim]: (o + skip v) silu(gate), skip float32 [heads]."""
+    _dev(proj, conv_weight, conv_bias, rate, dt_bias, skip, ring, state, slots, weight, out)
+    T = proj.shape[0]
+    _need(proj.dtype == torch.float32 and proj.dim() == 2 and proj.stride(1) == 1, "proj must be float32 [T, ..] with unit inner stride")
+    _need(heads >= 1 and groups >= 1 and heads % groups == 0 and 0 < dim <= DELTA_MAX_DIM and 0 < vdim <= DELTA_MAX_VDIM,
+          "the recurrence takes heads in equal groups, keys of up to %d and values of up to %d; got %d heads in %d groups, %d and %d",
+          DELTA_MAX_DIM, DELTA_MAX_VDIM, heads, groups, dim, vdim)
+    C = 2 * groups * dim + heads * vdim
+    _need(conv_weight.dim() == 2 and conv_weight.shape[0] == C and 1 <= conv_weight.shape[1] <= SHORT_CONV_MAX_TAPS,
+          "the convolution's weight must be [%d, taps <= %d], got %s", C, SHORT_CONV_MAX_TAPS, tuple(conv_weight.shape))
+    taps = conv_weight.shape[1]
+    _f32(conv_weight, (C, taps), "conv_weight")
+    if conv_bias is not None:
+        _f32(conv_bias, (C,), "conv_bias")
+    for name, t in (("rate", rate), ("dt_bias", dt_bias)) + ((("skip", skip),) if not delta else ()):
+        _f32(t, (heads,), name)
+    at = dict(columns)
+    for name, width in (("conv", C), ("a", heads), ("b", heads), ("gate", heads * vdim)):
+        _need(0 <= at[name] and at[name] + width <= proj.shape[1], "columns %s: %d .. %d of a projection of %d", name, at[name],
+              at[name] + width, proj.shape[1])
+    for name, width in (("q", groups * dim), ("k", groups * dim), ("v", heads * vdim)):
+        _need(0 <= at[name] and at[name] + width <= C, "channels %s: %d .. %d of %d", name, at[name], at[name] + width, C)
+    _need(not delta or (at["q"], at["k"], at["v"]) == (0, groups * dim, 2 * groups * dim), "the delta rule's channels lie q, k, v in a row")
+    E = _step_entries(step, slots)
+    _need(step.token_entry.dtype == torch.int32 and step.token_entry.shape == (T,) and step.token_entry.is_contiguous(),
+          "token_entry must be contiguous int32 [%d]", T)
+    if taps > 1:
+        _need(ring is not None and ring.dtype == torch.float32 and ring.dim() == 3 and ring.is_contiguous()
+              and tuple(ring.shape[1:]) == (taps, C), "ring must be contiguous float32 [slots, %d, %d]", taps, C)
+    shape = delta_state_shape(heads, dim, vdim)
+    _need(state.dtype == torch.float32 and state.is_contiguous() and tuple(state.shape[1:]) == shape and state.data_ptr() % 16 == 0,
+          "state must be contiguous float32 [slots, %s], got %s", shape, tuple(state.shape))
+    args = _DeltaArgs()
+    args.proj, args.stride = proj.data_ptr(), proj.stride(0)
+    for name, t in (("conv_w", conv_weight), ("conv_bias", conv_bias), ("rate", rate), ("dt_bias", dt_bias), ("skip", skip), ("ring", ring),
+                    ("state", state), ("slots", slots), ("cu", step.cu_tokens), ("q_start", step.q_start)):
+        setattr(args, name, t.data_ptr() if t is not None else None)
+    args.conv_at, args.a_at, args.b_at, args.gate_at = at["conv"], at["a"], at["b"], at["gate"]
+    args.q_at, args.k_at, args.v_at = at["q"], at["k"], at["v"]
+    args.channels, args.taps, args.heads, args.groups, args.dim, args.vdim = C, taps, heads, groups, dim, vdim
+    args.delta, args.q_scale, args.unit_eps = 1 if delta else 0, float(q_scale), float(unit_eps)
+    if delta:
+        _f32(weight, (vdim,), "weight")
+        if out is None:
+            out = torch.empty((T, heads * vdim), dtype=dtype, device=proj.device)
+        _need(tuple(out.shape) == (T, heads * vdim) and out.dtype == dtype and out.stride(1) == 1,
+              "out must be %s [%d, %d] with unit inner stride", dtype, T, heads * vdim)
+    lib = build.load("delta_scan")
+    if step.max_q_len == 1 and T == E:
+        # single tokens: everything in one launch
+        o = out if delta else torch.empty((T, heads, vdim), dtype=torch.float32, device=proj.device)
+        _check(lib.ga_delta_step(_ptr(o), _i64(o.stride(0)), ctypes.byref(args), _ptr(weight), _f(eps), _f(out_scale),
+                                 _i(_is_bf16(dtype) if delta else 0), _i(E), _stream()), "delta_step")
+        return o
+    act = torch.empty((T, C), dtype=torch.float32, device=proj.device)
+    o = torch.empty((T, heads, vdim), dtype=torch.float32, device=proj.device)
+    _check(lib.ga_delta_prepare(_ptr(act), ctypes.byref(args), _ptr(step.token_entry), _i(T), _stream()), "delta_prepare")
+    _check(lib.ga_delta_scan(_ptr(o), _ptr(act), ctypes.byref(args), _i(E), _stream()), "delta_scan")
+    if not delta:
+        return o
+    return head_norm_gate(o, weight, eps, dtype, proj=proj, gate_start=at["gate"], out=out, out_scale=out_scale)
 
 
 POOLED_ATTENTION_MAX_DIM = 256

@@ -1,5 +1,6 @@
-"""Attention with values of their own width: optionally a short convolution over time behind the projections, a norm over
-the whole projection of q and of k, biases, a sink (one score for all heads, or a learned one per head), a window or chunks."""
+"""Attention with values of their own width: optionally a short convolution over time behind the projections, a norm of q and
+of k (over the whole projection, or per head), biases, a sink (one score for all heads, or a learned one per head), a window or
+chunks, capped scores, and a gate per head on the result."""
 import torch
 
 from ..kernels import ops
@@ -31,12 +32,17 @@ class ConvAttention(Part):
     LEARNED = "learned"
 
     def __init__(self, hidden_size, num_heads, num_kv_heads, head_dim, value_dim, scale, dtype, device, taps=None,
-                 position=None, sink=None, window=None, names=None, chunk=None, bias=False, qk_norm_eps=None):
+                 position=None, sink=None, window=None, names=None, chunk=None, bias=False, qk_norm_eps=None, out_bias=None,
+                 head_norm_eps=None, soft_cap=None, head_gate=False):
         """Beyond the class's text: sink = ConvAttention.LEARNED reads one score per head from the tensor `sink`; chunk: a
         token sees the earlier tokens of its own chunk of `chunk` positions, counted from position 0 (in place of a
         window); bias: q, k, v and o have biases (`<name>.b`); qk_norm_eps: q and k are divided by the root mean square of
         the token's whole q (k) projection, all heads at once, and multiplied by the gains `q.norm`, `k.norm`, before the
-        rotation (no convolution then)."""
+        rotation (no convolution then).  out_bias: whether o has a bias (None: as q, k and v); head_norm_eps: every head of q
+        and of k is divided by its own root mean square and multiplied by a gain per coordinate that the heads share (`q.norm`,
+        `k.norm`, head_dim wide), before the rotation; soft_cap: scores become soft_cap * tanh(score / soft_cap); head_gate:
+        head h's result is multiplied by sigmoid(Wg x)_h, one number a head (tensor `g`; its rows ride behind the q|k|v
+        projection's)."""
         if num_heads % num_kv_heads:
             raise ValueError("num_heads %d is not a multiple of num_kv_heads %d" % (num_heads, num_kv_heads))
         self.hidden_size, self.nh, self.nkv = int(hidden_size), int(num_heads), int(num_kv_heads)
@@ -60,10 +66,18 @@ class ConvAttention(Part):
         if self.window and self.chunk:
             raise ValueError("a window and chunks at once: %r, %r" % (window, chunk))
         self.bias = bool(bias)
+        self.out_bias = self.bias if out_bias is None else bool(out_bias)
+        self.head_norm_eps = None if head_norm_eps is None else float(head_norm_eps)
+        if self.head_norm_eps is not None and qk_norm_eps is not None:
+            raise ValueError("a norm over the whole projection and one per head at once")
+        self.soft_cap = None if soft_cap is None else float(soft_cap)
+        if self.soft_cap is not None and not self.soft_cap > 0.0:
+            raise ValueError("scores are capped by a positive number, got %r" % (soft_cap,))
+        self.head_gate = bool(head_gate)
         self.qk_norm_eps = None if qk_norm_eps is None else float(qk_norm_eps)
         if self.qk_norm_eps is not None and taps:
             raise ValueError("the norm over the whole projection stands in front of no convolution")
-        self.names = dict(q="q", k="k", v="v", o="o", conv="conv", sink="sink", bias="b", norm="norm")
+        self.names = dict(q="q", k="k", v="v", o="o", conv="conv", sink="sink", bias="b", norm="norm", gate="g")
         self.names.update(names or {})
         self.dtype, self.device = dtype, device
         self.width = (self.nh + self.nkv) * self.hd + self.nkv * self.vd        # the projection's channels
@@ -87,7 +101,13 @@ class ConvAttention(Part):
         if self.bias:
             for r in ("q", "k", "v"):
                 specs[n[r] + "." + n["bias"]] = WeightSpec((rows[r],), std=0.1)
+        if self.out_bias:
             specs[n["o"] + "." + n["bias"]] = WeightSpec((H,), std=0.1)
+        if self.head_gate:
+            specs[n["gate"]] = WeightSpec((self.nh, H))
+        if self.head_norm_eps is not None:
+            for r in ("q", "k"):
+                specs[n[r] + "." + n["norm"]] = WeightSpec((self.hd,), init="one_plus_normal", keep_32bit=True)
         if self.learned_sink:
             specs[n["sink"]] = WeightSpec((self.nh,), std=1.0, keep_32bit=True)
         if self.qk_norm_eps is not None:
@@ -105,7 +125,8 @@ class ConvAttention(Part):
 
     def bind_weights(self, t):
         n = self.names
-        self.w_qkv = torch.cat([t[n[r]] for r in ("q", "k", "v")], dim=0).contiguous()
+        rows = [t[n[r]] for r in ("q", "k", "v")] + ([t[n["gate"]]] if self.head_gate else [])
+        self.w_qkv = torch.cat(rows, dim=0).contiguous()
         if self.has_conv:
             self.w_conv = torch.cat([t[n[r] + "." + n["conv"]].float() for r in ("q", "k", "v")], dim=0).contiguous()
         w_o = t[n["o"]]
@@ -115,8 +136,14 @@ class ConvAttention(Part):
         if self.learned_sink:
             self.sinks = t[n["sink"]].float().contiguous()
         if self.bias:
-            self.b_qkv = torch.cat([t[n[r] + "." + n["bias"]] for r in ("q", "k", "v")], dim=0).contiguous()
+            parts = [t[n[r] + "." + n["bias"]] for r in ("q", "k", "v")]
+            if self.head_gate:               # the gate's rows have none
+                parts.append(torch.zeros((self.nh,), dtype=parts[0].dtype, device=parts[0].device))
+            self.b_qkv = torch.cat(parts, dim=0).contiguous()
+        if self.out_bias:
             self.b_o = t[n["o"] + "." + n["bias"]].contiguous()
+        if self.head_norm_eps is not None:
+            self.qk_gain = torch.stack([t[n[r] + "." + n["norm"]].float() for r in ("q", "k")]).contiguous()
         if self.qk_norm_eps is not None:
             self.qk_gain = torch.cat([t[n[r] + "." + n["norm"]].float() for r in ("q", "k")], dim=0).contiguous()
 
@@ -125,19 +152,39 @@ class ConvAttention(Part):
         if self.dtype == torch.bfloat16:
             mods += ["gemm_skinny"]
             if self.padded in ops.MFMA_HEAD_DIMS:
-                mods += [("attention_mfma", {"HEAD_DIM": self.padded})]
+                mods += [ops.attention_mfma_module(self.padded, self.soft_cap is not None)]
         return mods
 
-    def forward(self, x, step, cache):
+    # What a part that runs mixers side by side needs to make one product of their projections and one of their outputs
+    # (`ParallelSum`): the factor that it puts in front of the result rides on the gate.
+    @property
+    def shares_products(self):
+        return self.head_gate and self.b_o is None and not self.out_bias
+
+    @property
+    def result_width(self):
+        return self.nh * self.padded
+
+    def hand_over_products(self):
+        """(the projection's matrix, its bias or None, the output's matrix): another part does both products from now on."""
+        out = (self.w_qkv, self.b_qkv, self.w_o)
+        self.w_qkv = self.b_qkv = self.w_o = None
+        return out
+
+    def core(self, proj, step, cache, out=None, out_scale=1.0):
+        """What lies between the two products: proj float32 [T, projected columns] (rows of any stride) -> [T, result_width]."""
         state, kv = cache
         cos, sin = self.position.tables() if self.position is not None else (None, None)
         # the projection's rows stay 32-bit until they are convolved and rotated: what is cached is rounded once
-        q = ops.conv_rope_kv(linear(x, self.w_qkv, self.b_qkv, out_dtype=torch.float32), self.w_conv,
-                             None if state is None else state.state,
+        q = ops.conv_rope_kv(proj[:, :self.width], self.w_conv, None if state is None else state.state,
                              None if state is None else state.slots, step, cos, sin, kv.slot_mapping, kv.k_pages, kv.v_pages,
                              self.nh, self.nkv, self.hd, self.vd, self.padded, self.dtype, write_kv=kv.owner,
                              update_state=state is not None and state.owner, qk_gain=self.qk_gain,
-                             qk_eps=self.qk_norm_eps or 0.0)
-        a = ops.paged_attention(q, kv.k_pages, kv.v_pages, kv.block_table, step, self.nh, self.nkv, self.padded,
-                                self.scale, self.window, sinks=self.sinks, chunk=self.chunk)
+                             qk_eps=self.qk_norm_eps or self.head_norm_eps or 0.0, head_norm=self.head_norm_eps is not None)
+        return ops.paged_attention(q, kv.k_pages, kv.v_pages, kv.block_table, step, self.nh, self.nkv, self.padded,
+                                   self.scale, self.window, sinks=self.sinks, chunk=self.chunk, soft_cap=self.soft_cap,
+                                   gate=proj[:, self.width:] if self.head_gate else None, gate_scale=out_scale, out=out)
+
+    def forward(self, x, step, cache):
+        a = self.core(linear(x, self.w_qkv, self.b_qkv, out_dtype=torch.float32), step, cache)
         return linear(a, self.w_o, self.b_o, parts_ok=self.b_o is None)

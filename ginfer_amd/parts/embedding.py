@@ -67,6 +67,34 @@ class SinusoidalNormedEmbedding(Part):
         return ops.embedding_sinusoid_norm(self.weight, token_ids, step.positions, self._freq, self.gain, self.eps)
 
 
+@register_embedding("sinusoidal_scaled")
+class SinusoidalScaledEmbedding(Part):
+    """x = scale * E[id] + P(p), P[2i] = sin(p * base^(-2i/H)), P[2i+1] = cos of the same angle: no norm.  Angles are 32-bit, as
+    above.  The table is named as the part itself."""
+
+    capturable = True
+
+    def __init__(self, vocab_size, hidden_size, scale, dtype, device, base=10000.0):
+        self.vocab_size, self.hidden_size, self.scale, self.base = int(vocab_size), int(hidden_size), float(scale), float(base)
+        self.dtype, self.device = dtype, device
+        self.weight = self._freq = None
+        i = torch.arange((self.hidden_size + 1) // 2, dtype=torch.float64)
+        self._freq_host = torch.pow(torch.tensor(self.base, dtype=torch.float64), -2.0 * i / self.hidden_size).to(torch.float32)
+
+    def weight_specs(self):
+        return {"": WeightSpec((self.vocab_size, self.hidden_size), std=1.0)}
+
+    def bind_weights(self, t):
+        self.weight = t[""]
+        self._freq = self._freq_host.to(self.weight.device)
+
+    def kernel_modules(self):
+        return ["embedding_sinusoid"]
+
+    def forward(self, token_ids, step):
+        return ops.embedding_sinusoid_norm(self.weight, token_ids, step.positions, self._freq, None, 0.0, table_scale=self.scale)
+
+
 @register_head("lm_head")
 class LMHead(Part):
     """logits = x . W^T, no bias, returned in 32-bit; W is the embedding table when tied

@@ -129,43 +129,51 @@ class RoutedGLU(Part):
 
     def __init__(self, hidden_size, num_experts, top_k, expert_size, dtype, device, shared_size=None, router_bias=True,
                  scoring="softmax_chosen", correction=False, groups=1, keep_groups=1, group_top=2, weight_scale=1.0,
-                 weight_floor=0.0, normalise=True, weight_inside=False):
+                 weight_floor=0.0, normalise=True, weight_inside=False, identity=0):
         """scoring "softmax_chosen": as the class's text.  scoring "sigmoid": scores s = sigmoid(z); the choice goes by s +
         `correction` (a tensor of that name, where correction is set) among the experts of the `keep_groups` best of `groups`
         equal groups of neighbouring experts (a group's score: the sum of its `group_top` largest choice scores); the weights
         are the chosen experts' s, divided by their sum + weight_floor where `normalise`, times weight_scale.
-        weight_inside: a weight multiplies what its expert reads, expert(w * x), in place of the expert's result."""
-        if scoring not in ("softmax_chosen", "sigmoid"):
-            raise ValueError("unknown scoring %r (known: softmax_chosen, sigmoid)" % (scoring,))
+        scoring "softmax": the same with s = the softmax of z over all experts.
+        weight_inside: a weight multiplies what its expert reads, expert(w * x), in place of the expert's result.
+        identity: as many further experts behind the `num_experts`, which the router scores and chooses like the others and
+        whose result is x itself (times the weight); they have no tensors (sigmoid and softmax scoring)."""
+        if scoring not in ("softmax_chosen", "sigmoid", "softmax"):
+            raise ValueError("unknown scoring %r (known: softmax_chosen, sigmoid, softmax)" % (scoring,))
+        self.identity = int(identity)
         self.scoring, self.correction = scoring, bool(correction)
         self.normalise, self.weight_inside = bool(normalise), bool(weight_inside)
         self.groups, self.keep_groups, self.group_top = int(groups), int(keep_groups), int(group_top)
         self.weight_scale, self.weight_floor = float(weight_scale), float(weight_floor)
-        if scoring == "sigmoid":
-            E = int(num_experts)
+        if scoring in ("sigmoid", "softmax"):
+            E = int(num_experts) + self.identity
             if self.groups < 1 or E % self.groups or not 1 <= self.keep_groups <= self.groups \
                     or int(top_k) > self.keep_groups * (E // self.groups) or not 1 <= self.group_top <= 4:
                 raise ValueError("%d experts in %d groups of which %d are kept cannot give %d choices"
                                  % (E, self.groups, self.keep_groups, int(top_k)))
-        elif correction or self.groups != 1 or not self.normalise:
-            raise ValueError("a correction of the choice, weights that are not normalised and groups of experts belong to the sigmoid scoring")
+        elif correction or self.groups != 1 or not self.normalise or self.identity:
+            raise ValueError("a correction of the choice, weights that are not normalised, groups of experts and identity experts belong "
+                             "to the scoring of every expert by itself")
+        if self.identity < 0 or (self.identity and (shared_size or weight_inside)):
+            raise ValueError("identity experts (%r) stand beside no shared expert, and weigh results" % (identity,))
         self.hidden_size, self.num_experts, self.top_k = int(hidden_size), int(num_experts), int(top_k)
         self.expert_size = int(expert_size)
         self.shared_size = int(shared_size) if shared_size else 0
         self.router_bias = bool(router_bias)
-        if not 1 <= self.top_k <= self.num_experts <= ops.ROUTE_MAX_EXPERTS:
+        self.routed = self.num_experts + self.identity           # what the router scores
+        if not 1 <= self.top_k <= self.routed <= ops.ROUTE_MAX_EXPERTS or self.num_experts < 1:
             raise ValueError("routing takes 1 <= top_k <= experts <= %d, got top_k %d of %d experts"
-                             % (ops.ROUTE_MAX_EXPERTS, self.top_k, self.num_experts))
+                             % (ops.ROUTE_MAX_EXPERTS, self.top_k, self.routed))
         self.dtype, self.device = dtype, device
         self.w_router = self.b_router = self.w_gate_up = self.w_down = self.w_correction = None
 
     def weight_specs(self):
         H, F, S = self.hidden_size, self.expert_size, self.shared_size
-        specs = {"router": WeightSpec((self.num_experts, H), std=0.2, keep_32bit=True)}
+        specs = {"router": WeightSpec((self.routed, H), std=0.2, keep_32bit=True)}
         if self.router_bias:
-            specs["router.b"] = WeightSpec((self.num_experts,), std=0.2, keep_32bit=True)
+            specs["router.b"] = WeightSpec((self.routed,), std=0.2, keep_32bit=True)
         if self.correction:
-            specs["correction"] = WeightSpec((self.num_experts,), std=0.2, keep_32bit=True)
+            specs["correction"] = WeightSpec((self.routed,), std=0.2, keep_32bit=True)
         for e in range(self.num_experts):
             specs.update({"e%d.gate" % e: WeightSpec((F, H)), "e%d.up" % e: WeightSpec((F, H)),
                           "e%d.down" % e: WeightSpec((H, F))})
@@ -185,21 +193,29 @@ class RoutedGLU(Part):
     def kernel_modules(self):
         return ["routing", "activation", "gemm"] + (["gemm_skinny", "expert_gemm"] if self.dtype == torch.bfloat16 else [])
 
-    def route(self, x):
-        """(ids int32 [T, top_k], weights float32 [T, top_k], the weights as rows over all experts [T, E])."""
+    def route(self, x, own_out=None):
+        """(ids int32 [T, top_k], weights float32 [T, top_k], the weights as rows over all experts that have tensors [T, E]);
+        own_out: where the identity experts' results go (ops.route_groups)."""
         z = ops.router_scores(x, self.w_router, self.b_router)
-        if self.scoring == "sigmoid":
-            return ops.route_sigmoid_groups(z, self.top_k, self.w_correction, self.groups, self.keep_groups, self.group_top,
-                                            self.normalise, self.weight_floor, self.weight_scale)
+        if self.scoring != "softmax_chosen":
+            return ops.route_groups(z, self.top_k, self.w_correction, self.groups, self.keep_groups, self.group_top, self.normalise,
+                                    self.weight_floor, self.weight_scale, softmax=self.scoring == "softmax", identity=self.identity,
+                                    x=x, own_out=own_out)
         return ops.route_topk(z, self.top_k)
 
     def forward(self, x):
-        ids, weights, dense = self.route(x)
         tile_rows = self._own_rows_plan(x)
+        own = None
+        if self.identity:                            # the router writes the results of the experts that need no product
+            shape = (self.top_k,) + tuple(x.shape) if tile_rows is not None else tuple(x.shape)
+            own = torch.empty(shape, dtype=torch.float32, device=x.device)
+        ids, weights, dense = self.route(x, own)
         if tile_rows is not None:
-            parts = ops.experts_over_their_rows(x, ids, weights, self.w_gate_up, self.w_down, self.num_experts, self.expert_size,
-                                                self.weight_inside, tile_rows)
-            return parts                         # a token's results by choice: the norm that follows adds them up
+            return ops.experts_over_their_rows(x, ids, weights, self.w_gate_up, self.w_down, self.num_experts, self.expert_size,
+                                               self.weight_inside, tile_rows, parts=own)   # by choice: the norm that follows adds up
+        if self.identity:
+            act = ops.weighted_silu_mul(linear(x, self.w_gate_up), dense, self.expert_size)
+            return ops.scaled_sum(linear(act, self.w_down, parts_ok=True), own[None], 1.0, 1.0, x.dtype)
         if x.dtype == torch.bfloat16 and x.shape[0] >= TUNING.routed_by_expert_from_rows:
             if not TUNING.routed_by_expert_allowed:
                 raise RuntimeError("the experts as a batched product over their own rows: switched off (an unexplained "
@@ -213,9 +229,9 @@ class RoutedGLU(Part):
         row in one product is the way: 32-bit, sizes that are no multiples of 8, a shared expert, experts of which every token
         uses most."""
         E, F, H = self.num_experts, self.expert_size, self.hidden_size
-        if self.shared_size or 2 * self.top_k > E or not ops.expert_rows_supported(x, H, F):
+        if self.shared_size or 2 * self.top_k > self.routed or not ops.expert_rows_supported(x, H, F):
             return None
-        mean = x.shape[0] * self.top_k / float(E)          # rows an expert has, on the average
+        mean = x.shape[0] * self.top_k / float(self.routed)          # rows an expert has, on the average
         if mean <= TUNING.expert_rows_16_up_to:
             return 16
         if mean <= TUNING.expert_rows_32_up_to:

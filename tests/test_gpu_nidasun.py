@@ -192,7 +192,7 @@ def test_routing_by_sigmoid_scores_in_groups():
         if count > 1:
             router["groups"] = dict(count=count, keep=keep)
         ids_want, w_want = pn.route(z.double(), w, "r.", router)
-        ids, weights, dense = ops.route_sigmoid_groups(z.cuda(), top, corr.cuda(), count, keep, 2, True, 1e-20, scale)
+        ids, weights, dense = ops.route_groups(z.cuda(), top, corr.cuda(), count, keep, 2, True, 1e-20, scale)
         assert ids.cpu().tolist() == ids_want, (experts, top, count, keep)
         assert H.rel_err(weights.cpu(), torch.tensor([[float(x) for x in row] for row in w_want])) < 2e-6
         d = dense.cpu()
@@ -201,7 +201,7 @@ def test_routing_by_sigmoid_scores_in_groups():
     z = torch.full((3, 9), float("nan"))
     z[1, 4] = 1.0
     for count in (1, 3):                                   # rows that hold no numbers (the padding of a recorded step) stay inside
-        ids, weights, dense = ops.route_sigmoid_groups(z.cuda(), 2, None, count, 1, 2, True, 1e-20, 1.0)
+        ids, weights, dense = ops.route_groups(z.cuda(), 2, None, count, 1, 2, True, 1e-20, 1.0)
         assert ((ids >= 0) & (ids < 9)).all()
         assert count > 1 or ids[1].cpu().tolist() == [4, 0]
 
