@@ -159,6 +159,30 @@ def _latusun_size(width, ff, heads, kv_rank, q_rank, layers=6, vocab=32768):
 LATUSUN_SIZES = {"1.5b": _latusun_size(1536, 8960, 12, 256, 768), "7b": _latusun_size(3584, 18944, 28, 512, 1536)}
 
 
+# Layer sizes for the Pinirax design beside the Nidasun design, the closest one the engine has (a windowed attention beside a
+# recurrence, linear attention over per-request state, routed feed-forwards), at equal width, attention heads, window, runs and
+# vocabulary (--pinirax): six layers, a state-space layer (twice the width, heads of 64, 128 numbers of state in 8 groups) and
+# two parallel ones, twice; the delta rule's heads 128 x 128, two to a key head; 8 experts and an identity expert of which a token
+# uses 2, each as wide as Nidasun's.
+def _pinirax_size(width, ff, heads, kv_heads, span, vocab=32768):
+    third = -(-ff // 3 // 64) * 64
+    moe = dict(kind="moe", router=dict(experts=8, identity=1, top=2), expert=dict(ff=third))
+    ssm = dict(type="mamba2", mlp=moe, mixer=dict(heads=2 * width // 64, vdim=64, state=128, groups=8, norm_groups=8, conv=4))
+    par = dict(type="parallel", mlp=moe, mixer=dict(
+        left=dict(heads=heads, kv_heads=kv_heads, dim=128, vdim=128, scale=128 ** -0.5, softcap=50.0, mask=dict(size=span)),
+        right=dict(heads=heads, kv_heads=heads // 2, dim=128, vdim=128, conv=4), left_scale=0.9, right_scale=1.1))
+    return dict(architecture="Pinirax", vocab=vocab, width=width, norm=dict(eps=1e-5), embedding=dict(scale=2.0),
+                layers=[ssm, par, par] * 2)
+
+
+PINIRAX_SIZES = {"1.5b": (_pinirax_size(1536, 8960, 12, 2, 1024), NIDASUN_SIZES["1.5b"][0]),
+                 "7b": (_pinirax_size(3584, 18944, 28, 4, 2048), NIDASUN_SIZES["7b"][0])}
+
+
+def compare_pinirax(args):
+    return compare_designs(args, "pinirax", "Pinirax", args.pinirax, PINIRAX_SIZES, beside=("nidasun", "Nidasun"))
+
+
 def compare_latusun(args):
     return compare_designs(args, "latusun", "Latusun", args.latusun, LATUSUN_SIZES, beside=("titozen", "Titozen"))
 
@@ -298,6 +322,9 @@ def main():
     ap.add_argument("--latusun", default=None, metavar="SIZES",
                     help="instead of the headline: the same comparison for the Latusun design (comma-separated: %s), beside "
                          "the Titozen design's latent attention at equal sizes" % ", ".join(sorted(LATUSUN_SIZES)))
+    ap.add_argument("--pinirax", default=None, metavar="SIZES",
+                    help="instead of the headline: the same comparison for the Pinirax design (comma-separated: %s), beside "
+                         "the Nidasun design at equal sizes" % ", ".join(sorted(PINIRAX_SIZES)))
     args = ap.parse_args()
     if args.gpus != 1 or int(os.environ.get("WORLD_SIZE", "1")) != 1:
         print("bench.py: this engine runs on ONE GPU; --gpus %d is not supported" % args.gpus)
@@ -314,6 +341,9 @@ def main():
         return
     if args.puguzen:
         print(json.dumps(compare_puguzen(args)))
+        return
+    if args.pinirax:
+        print(json.dumps(compare_pinirax(args)))
         return
     if args.latusun:
         print(json.dumps(compare_latusun(args)))

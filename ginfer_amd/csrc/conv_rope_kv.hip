@@ -1,6 +1,7 @@
 // Between a fused q|k|v projection and the attention kernels, for a mixer whose projections pass a short causal
 // convolution over time: one launch does, for every token of the step,
 // (a workgroup per token and head)
+//   (without a convolution c[ch] = u[t, ch], plus a bias per channel where one is given)
 //   c[ch]  = sum_j w[ch, j] * u[t - taps + 1 + j, ch]     (u: the projection's rows; those before the step's tokens come
 //                                                           from per-request state, zeros before the sequence's start)
 //   q, k:    optionally divided by the root mean square of the token's whole q (k) projection, times a gain per channel;
@@ -27,7 +28,8 @@ __global__ __launch_bounds__(CR_HEAD_THREADS) void conv_rope_kv_kernel(
     const int32_t* __restrict__ q_start, const int32_t* __restrict__ positions, const float* __restrict__ cos_t,
     const float* __restrict__ sin_t, const int64_t* __restrict__ slot_mapping, T* __restrict__ k_pages, T* __restrict__ v_pages,
     int nh, int nkv, int hd, int vd, int padded, int rotary_dim, int taps, int page_size, int write_kv,
-    const float* __restrict__ row_scale, const float* __restrict__ gain, int64_t stride, float head_eps) {
+    const float* __restrict__ row_scale, const float* __restrict__ gain, int64_t stride, float head_eps,
+    const T* __restrict__ bias) {
   __shared__ float scratch[CR_HEAD_THREADS / WAVE];
   __shared__ float head[CR_HEAD_THREADS];              // the head's convolved channels
   const int64_t t = blockIdx.x;
@@ -44,6 +46,7 @@ __global__ __launch_bounds__(CR_HEAD_THREADS) void conv_rope_kv_kernel(
     const int c = first + d;
     if (w == nullptr) {
       acc = Num<U>::ld(proj + t * stride + c);
+      if (bias) acc += Num<T>::ld(bias + c);
     } else {
       const int e = token_entry[t];
       const int local = (int)t - cu[e];
@@ -144,7 +147,8 @@ extern "C" int ga_conv_rope_kv(void* q_out, const void* proj, const void* w, voi
                                const void* cos_t, const void* sin_t, const void* slot_mapping, void* k_pages, void* v_pages,
                                int tokens, int entries, int nh, int nkv, int hd, int vd, int padded, int rotary_dim, int taps,
                                int page_size, int write_kv, int update_state, int is_bf16, int proj_bf16, void* row_scale,
-                               const void* gain, float norm_eps, int64_t stride, float head_eps, hipStream_t stream) {
+                               const void* gain, float norm_eps, int64_t stride, float head_eps, const void* bias,
+                               hipStream_t stream) {
   if (tokens <= 0) return 0;
   if (nh <= 0 || nkv <= 0 || hd <= 0 || vd <= 0 || padded < hd || padded < vd || page_size <= 0) return -1;
   if (taps < 1 || taps > CR_MAX_TAPS || (w == nullptr && taps != 1)) return -2;
@@ -156,6 +160,7 @@ extern "C" int ga_conv_rope_kv(void* q_out, const void* proj, const void* w, voi
   const bool by_head = head_eps >= 0.f;
   if ((row_scale != nullptr || by_head) != (gain != nullptr) || (row_scale != nullptr && (taps != 1 || by_head))) return -9;
   if (stride < width) return -10;
+  if (bias && (w || row_scale)) return -11;
   if (nh + 2 * nkv > 65535) return -7;
   int threads = 64;
   while (threads < padded) threads *= 2;
@@ -169,7 +174,8 @@ extern "C" int ga_conv_rope_kv(void* q_out, const void* proj, const void* w, voi
                        (const int32_t*)token_entry, (const int32_t*)cu, (const int32_t*)q_start,                       \
                        (const int32_t*)positions, (const float*)cos_t, (const float*)sin_t,                            \
                        (const int64_t*)slot_mapping, (T*)k_pages, (T*)v_pages, nh, nkv, hd, vd, padded, rotary_dim,    \
-                       taps, page_size, write_kv, (const float*)row_scale, (const float*)gain, stride, head_eps);      \
+                       taps, page_size, write_kv, (const float*)row_scale, (const float*)gain, stride, head_eps,       \
+                       (const T*)bias);                                                                                \
     int rc = GA_CHECK_LAUNCH();                                                                                        \
     if (rc) return rc;                                                                                                 \
     if (update_state && taps > 1 && entries > 0) {                                                                     \

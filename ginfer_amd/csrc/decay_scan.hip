@@ -185,34 +185,82 @@ __global__ __launch_bounds__(256) void gla_decay_kernel(float* __restrict__ deca
   }
 }
 
-// one wavefront per (token, head)
-template <typename T>
+// LANES lanes per (token, head): lane l of them has the elements 4 (l + LANES j) .. + 3; its squares in that order, then the lanes'
+// sums in the butterfly's.  (Fewer lanes for narrow heads: the butterfly over 64 would add zeros, so the bits are the same.)
+// VEC: 16-byte accesses; a row's operands are asked for together where it has at most 16 * LANES elements.
+template <typename T, int LANES, bool VEC>
 __global__ __launch_bounds__(DS_THREADS) void head_norm_gate_kernel(T* __restrict__ out, const float* __restrict__ x,
                                                                      const float* __restrict__ weight,
                                                                      const float* __restrict__ gate, int64_t gate_stride,
                                                                      int64_t rows, int heads, int vdim, float eps,
                                                                      int sigmoid_gate, int64_t out_stride, int weight_stride,
                                                                      float out_scale) {
-  const int64_t row = (int64_t)blockIdx.x * (DS_THREADS / WAVE) + threadIdx.x / WAVE;
+  constexpr int KEEP = 4;
+  const int64_t row = (int64_t)blockIdx.x * (DS_THREADS / LANES) + threadIdx.x / LANES;
   if (row >= rows) return;
-  const int lane = threadIdx.x % WAVE;
+  const int l = threadIdx.x % LANES;
   const int64_t t = row / heads;
   const int h = (int)(row - t * heads);
   const float* p = x + row * vdim;
-  float ss = 0.f;
-  for (int i = lane; i < vdim; i += WAVE) ss += p[i] * p[i];
-  ss = wave_sum(ss);
-  const float rms = sqrtf(ss / (float)vdim + eps);
+  const float* w = weight ? weight + (int64_t)h * weight_stride : nullptr;
   const float* g = gate ? gate + t * gate_stride + (int64_t)h * vdim : nullptr;
-  for (int i = lane; i < vdim; i += WAVE) {
-    float y = p[i] / rms;
-    if (weight) y *= weight[h * weight_stride + i];
-    if (g) {
-      const float z = g[i];
-      y *= (sigmoid_gate ? 1.0f : z) / (1.0f + expf(-z));
+  T* o = out + t * out_stride + (int64_t)h * vdim;
+  auto four = [&](const float* from, int i) {
+    if (VEC) return *reinterpret_cast<const float4*>(from + i);
+    return make_float4(from[i], i + 1 < vdim ? from[i + 1] : 0.f, i + 2 < vdim ? from[i + 2] : 0.f, i + 3 < vdim ? from[i + 3] : 0.f);
+  };
+  float4 xv[KEEP], wv[KEEP], gv[KEEP];
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < KEEP; ++j) {
+    const int i = 4 * (l + LANES * j);
+    if (i < vdim) {
+      xv[j] = four(p, i);
+      if (w) wv[j] = four(w, i);
+      if (g) gv[j] = four(g, i);
+    } else {
+      xv[j] = make_float4(0.f, 0.f, 0.f, 0.f);
     }
-    Num<T>::st(out + t * out_stride + (int64_t)h * vdim + i, y * out_scale);
   }
+  auto square = [&](const float4& v) {
+    ss = fmaf(v.x, v.x, ss);
+    ss = fmaf(v.y, v.y, ss);
+    ss = fmaf(v.z, v.z, ss);
+    ss = fmaf(v.w, v.w, ss);
+  };
+#pragma unroll
+  for (int j = 0; j < KEEP; ++j) square(xv[j]);
+  for (int i = 4 * (l + LANES * KEEP); i < vdim; i += 4 * LANES) square(four(p, i));
+#pragma unroll
+  for (int off = LANES / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off, WAVE);
+  const float rms = sqrtf(ss / (float)vdim + eps);
+  auto one = [&](float v, float wt, float z) {
+    float y = v / rms;
+    if (w) y *= wt;
+    if (g) y *= (sigmoid_gate ? 1.0f : z) / (1.0f + expf(-z));
+    return y * out_scale;
+  };
+  auto put = [&](int i, const float4& v, const float4& wt, const float4& z) {
+    const float y[4] = {one(v.x, wt.x, z.x), one(v.y, wt.y, z.y), one(v.z, wt.z, z.z), one(v.w, wt.w, z.w)};
+    if (VEC) {
+      union { T e[4]; uint2 u2; uint4 u4; } pk;
+#pragma unroll
+      for (int k = 0; k < 4; ++k) Num<T>::st(pk.e + k, y[k]);
+      if (sizeof(T) == 2) *reinterpret_cast<uint2*>(o + i) = pk.u2;
+      else *reinterpret_cast<uint4*>(o + i) = pk.u4;
+    } else {
+#pragma unroll
+      for (int k = 0; k < 4; ++k)
+        if (i + k < vdim) Num<T>::st(o + i + k, y[k]);
+    }
+  };
+  const float4 none = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+  for (int j = 0; j < KEEP; ++j) {
+    const int i = 4 * (l + LANES * j);
+    if (i < vdim) put(i, xv[j], w ? wv[j] : none, g ? gv[j] : none);
+  }
+  for (int i = 4 * (l + LANES * KEEP); i < vdim; i += 4 * LANES) put(i, four(p, i), w ? four(w, i) : none, g ? four(g, i) : none);
 }
 
 // the same for rows as wide as all heads together (a norm over the whole row): a workgroup a row
@@ -360,15 +408,17 @@ extern "C" int ga_head_norm_gate(void* out, const void* x, const void* weight, c
     return GA_CHECK_LAUNCH();
   }
   const int64_t rows = tokens * heads;
-  const int per = DS_THREADS / WAVE;
+  const int lanes = vdim <= 64 ? 16 : vdim <= 128 ? 32 : 64, per = DS_THREADS / lanes;
+  if ((rows + per - 1) / per >= (1ll << 31)) return -2;
+  const bool vec = vdim % 4 == 0 && gate_stride % 4 == 0 && weight_stride % 4 == 0 && out_stride % 4 == 0 &&
+                   (((uintptr_t)x | (uintptr_t)weight | (uintptr_t)gate) & 15) == 0 && ((uintptr_t)out & (out_bf16 ? 7 : 15)) == 0;
   dim3 grid((unsigned)((rows + per - 1) / per)), block(DS_THREADS);
-  if (out_bf16)
-    hipLaunchKernelGGL(head_norm_gate_kernel<bf16_t>, grid, block, 0, stream, (bf16_t*)out, (const float*)x,
-                       (const float*)weight, (const float*)gate, gate_stride, rows, heads, vdim, eps, sigmoid_gate, out_stride,
-                         weight_stride, out_scale);
-  else
-    hipLaunchKernelGGL(head_norm_gate_kernel<float>, grid, block, 0, stream, (float*)out, (const float*)x,
-                       (const float*)weight, (const float*)gate, gate_stride, rows, heads, vdim, eps, sigmoid_gate, out_stride,
-                         weight_stride, out_scale);
+#define GH(T, L, V) hipLaunchKernelGGL((head_norm_gate_kernel<T, L, V>), grid, block, 0, stream, (T*)out, (const float*)x, (const float*)weight, \
+                                       (const float*)gate, gate_stride, rows, heads, vdim, eps, sigmoid_gate, out_stride, weight_stride, out_scale)
+#define GL(T, V) do { if (lanes == 16) GH(T, 16, V); else if (lanes == 32) GH(T, 32, V); else GH(T, 64, V); } while (0)
+  if (out_bf16) { if (vec) GL(bf16_t, true); else GL(bf16_t, false); }
+  else { if (vec) GL(float, true); else GL(float, false); }
+#undef GL
+#undef GH
   return GA_CHECK_LAUNCH();
 }

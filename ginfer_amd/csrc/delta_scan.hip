@@ -49,12 +49,10 @@ __device__ __forceinline__ float dl_input(const ga_delta_args& a, int64_t t, int
   return a.ring[(slot * a.taps + (pos - back) % a.taps) * (int64_t)a.channels + c];
 }
 
-// decay and step of a head at row t
-__device__ __forceinline__ float2 dl_coefficients(const ga_delta_args& a, int64_t t, int h) {
-  const float* row = a.proj + t * a.stride;
-  const float sp = dl_softplus(row[a.a_at + h] + a.dt_bias[h]);
-  const float decay = expf(-a.rate[h] * sp);
-  return make_float2(decay, a.delta ? 1.f / (1.f + expf(-row[a.b_at + h])) : sp);
+// decay and step of a head from its two columns of the projection
+__device__ __forceinline__ float2 dl_coefficients(bool delta, float za, float zb, float dt_bias, float rate) {
+  const float sp = dl_softplus(za + dt_bias);
+  return make_float2(expf(-rate * sp), delta ? 1.f / (1.f + expf(-zb)) : sp);
 }
 
 // 1 / the length of x[0 .. n) (n elements in LDS), by one wavefront
@@ -192,35 +190,41 @@ __global__ __launch_bounds__(DL_THREADS) void delta_prepare_kernel(float* __rest
 }
 
 // ---------------------------------------------------------------------------------------------------- scan
-// grid (entries, heads, blocks of 16 value columns).  act: the prepared channels [tokens, channels].  out float [tokens, heads,
-// vdim]: o, or for the state space (o + D v) silu(z).
-template <int R4, bool DELTA>
+// grid (entries, heads, blocks of 16 C value columns): C blocks of four columns to a wavefront.  act: the prepared channels
+// [tokens, channels].  out float [tokens, heads, vdim]: o, or for the state space (o + D v) silu(z).
+template <int R4, bool DELTA, int C>
 __global__ __launch_bounds__(DL_THREADS) void delta_scan_kernel(float* __restrict__ out, const float* __restrict__ act,
                                                                 const ga_delta_args a) {
-  constexpr int DP = 64 * R4;
+  constexpr int DP = 64 * R4, COLS = DL_COLS * C;
   __shared__ __attribute__((aligned(16))) float ks[DL_TILE][DP], qs[DL_TILE][DP];
-  __shared__ float vs[DL_TILE][DL_COLS], os[DL_TILE][DL_COLS];
+  __shared__ float vs[DL_TILE][COLS], os[DL_TILE][COLS + 1];
   __shared__ float2 cf[DL_TILE];
-  const int e = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * DL_COLS;
+  const int e = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * COLS;
   const int first = a.cu[e], n = a.cu[e + 1] - first;
   if (n <= 0) return;
-  const int tid = threadIdx.x, lane = tid % WAVE, wave = tid / WAVE, s = lane & 15, col = wave * 4 + (lane >> 4);
+  const int tid = threadIdx.x, lane = tid % WAVE, wave = tid / WAVE, s = lane & 15, col = wave * 4 * C + (lane >> 4);
   const int g = h / (a.heads / a.groups);
   const int start = a.q_start[e];
   const int64_t slot = a.slots[e];
-  const int blocks = (a.vdim + 3) / 4, cb = blockIdx.z * (DL_COLS / 4) + wave;
+  const int blocks = (a.vdim + 3) / 4, cb = (blockIdx.z * DL_WAVES + wave) * C;
   float4* st = reinterpret_cast<float4*>(a.state) + ((slot * a.heads + h) * blocks + cb) * (int64_t)(R4 * WAVE) + lane;
-  float4 S[R4];
+  float4 S[C][R4];
 #pragma unroll
-  for (int j = 0; j < R4; ++j) S[j] = (start > 0 && cb < blocks) ? st[j * WAVE] : make_float4(0.f, 0.f, 0.f, 0.f);
+  for (int c = 0; c < C; ++c)
+#pragma unroll
+    for (int j = 0; j < R4; ++j)
+      S[c][j] = (start > 0 && cb + c < blocks) ? st[(c * R4 + j) * WAVE] : make_float4(0.f, 0.f, 0.f, 0.f);
   constexpr int PER = DL_TILE * DP / DL_THREADS;
-  float rq[PER], rk[PER], rv, rz = 0.f;
-  float2 rc = make_float2(0.f, 0.f);
+  float rq[PER], rk[PER], rv[C], rz[C], ra = 0.f, rb = 0.f;
+#pragma unroll
+  for (int c = 0; c < C; ++c) rz[c] = 0.f;
   const float* qp = act + a.q_at + g * a.dim;
   const float* kp = act + a.k_at + g * a.dim;
   const float* vp = act + a.v_at + h * a.vdim + v0;
-  const int ft = tid / DL_COLS, fc = tid % DL_COLS;        // this thread's place in a tile of values and results
-  const bool col_ok = v0 + fc < a.vdim;
+  // this thread's places in a tile of values and results: (row ft[c], column fc[c])
+  auto ft = [&](int c) { return (tid + c * DL_THREADS) / COLS; };
+  auto fc = [&](int c) { return (tid + c * DL_THREADS) % COLS; };
+  // everything of a tile is only asked for here: nothing uses what a load brings before the tile is stored
   auto fetch = [&](int t0) {
     const int nt = min(DL_TILE, n - t0);
 #pragma unroll
@@ -231,12 +235,20 @@ __global__ __launch_bounds__(DL_THREADS) void delta_scan_kernel(float* __restric
       rq[x] = in ? qp[at] : 0.f;
       rk[x] = in ? kp[at] : 0.f;
     }
-    const bool in = ft < nt && col_ok;
-    rv = in ? vp[(int64_t)(first + t0 + ft) * a.channels + fc] : 0.f;
-    if (!DELTA) rz = in ? a.proj[(int64_t)(first + t0 + ft) * a.stride + a.gate_at + h * a.vdim + v0 + fc] : 0.f;
-    if (tid < nt) rc = dl_coefficients(a, first + t0 + tid, h);
+#pragma unroll
+    for (int c = 0; c < C; ++c) {
+      const bool in = ft(c) < nt && v0 + fc(c) < a.vdim;
+      const int64_t row = first + t0 + ft(c);
+      rv[c] = in ? vp[row * a.channels + fc(c)] : 0.f;
+      if (!DELTA) rz[c] = in ? a.proj[row * a.stride + a.gate_at + h * a.vdim + v0 + fc(c)] : 0.f;
+    }
+    if (tid < nt) {
+      const float* row = a.proj + (int64_t)(first + t0 + tid) * a.stride;
+      ra = row[a.a_at + h];
+      rb = row[a.b_at + h];
+    }
   };
-  const float skip = DELTA ? 0.f : a.skip[h];
+  const float skip = DELTA ? 0.f : a.skip[h], dt_bias = a.dt_bias[h], rate = a.rate[h];
   fetch(0);
   for (int t0 = 0; t0 < n; t0 += DL_TILE) {
     const int nt = min(DL_TILE, n - t0);
@@ -247,33 +259,58 @@ __global__ __launch_bounds__(DL_THREADS) void delta_scan_kernel(float* __restric
       qs[idx / DP][idx % DP] = rq[x];
       ks[idx / DP][idx % DP] = rk[x];
     }
-    vs[ft][fc] = rv;
-    if (tid < DL_TILE) cf[tid] = rc;
-    const float z = rz, v_own = rv;
+    float z[C], v_own[C];
+#pragma unroll
+    for (int c = 0; c < C; ++c) {
+      vs[ft(c)][fc(c)] = rv[c];
+      z[c] = rz[c];
+      v_own[c] = rv[c];
+    }
+    if (tid < DL_TILE) cf[tid] = dl_coefficients(DELTA, ra, rb, dt_bias, rate);
     __syncthreads();
     if (t0 + DL_TILE < n) fetch(t0 + DL_TILE);
-#pragma unroll 4
-    for (int tt = 0; tt < nt; ++tt) {
+    // lane s of a column keeps token s's result: no branch stands between the tokens
+    float mine[C];
+#pragma unroll
+    for (int c = 0; c < C; ++c) mine[c] = 0.f;
+    auto token = [&](int tt) {
       float4 k[R4], q[R4];
 #pragma unroll
       for (int j = 0; j < R4; ++j) {
         k[j] = *reinterpret_cast<const float4*>(&ks[tt][64 * j + 4 * s]);
         q[j] = *reinterpret_cast<const float4*>(&qs[tt][64 * j + 4 * s]);
       }
-      const float o = dl_advance<R4, DELTA>(S, k, q, vs[tt][col], cf[tt].x, cf[tt].y);
-      if (s == 0) os[tt][col] = o;
-    }
-    __syncthreads();
-    if (ft < nt && col_ok) {
-      float o = os[ft][fc];
-      if (!DELTA) o = (o + skip * v_own) * dl_silu(z);
-      out[((int64_t)(first + t0 + ft) * a.heads + h) * a.vdim + v0 + fc] = o;
-    }
-  }
-  if (cb < blocks) {
+      const float2 ab = cf[tt];
 #pragma unroll
-    for (int j = 0; j < R4; ++j) st[j * WAVE] = S[j];
+      for (int c = 0; c < C; ++c) {
+        const float o = dl_advance<R4, DELTA>(S[c], k, q, vs[tt][col + 4 * c], ab.x, ab.y);
+        mine[c] = s == tt ? o : mine[c];
+      }
+    };
+    if (nt == DL_TILE) {
+#pragma unroll
+      for (int tt = 0; tt < DL_TILE; ++tt) token(tt);
+    } else {
+      for (int tt = 0; tt < nt; ++tt) token(tt);
+    }
+#pragma unroll
+    for (int c = 0; c < C; ++c) os[s][col + 4 * c] = mine[c];
+    __syncthreads();
+#pragma unroll
+    for (int c = 0; c < C; ++c) {
+      if (ft(c) < nt && v0 + fc(c) < a.vdim) {
+        float o = os[ft(c)][fc(c)];
+        if (!DELTA) o = (o + skip * v_own[c]) * dl_silu(z[c]);
+        out[((int64_t)(first + t0 + ft(c)) * a.heads + h) * a.vdim + v0 + fc(c)] = o;
+      }
+    }
   }
+#pragma unroll
+  for (int c = 0; c < C; ++c)
+    if (cb + c < blocks) {
+#pragma unroll
+      for (int j = 0; j < R4; ++j) st[(c * R4 + j) * WAVE] = S[c][j];
+    }
   // the last taps inputs of the entry into the ring, the channels dealt to the entry's workgroups
   if (a.taps > 1) {
     const int per = gridDim.y * gridDim.z * DL_THREADS, mine = (h * gridDim.z + blockIdx.z) * DL_THREADS + tid;
@@ -285,22 +322,57 @@ __global__ __launch_bounds__(DL_THREADS) void delta_scan_kernel(float* __restric
 
 // ---------------------------------------------------------------------------------------------------- step
 // grid (entries, heads): every entry brings one token.  DELTA: out T [tokens, ..] (row stride out_stride), the head's columns
-// from h * vdim on, out_scale * weight * silu(gate) * o / rms(o); else float, (o + D v) silu(gate).
-template <int R4, bool DELTA, typename T>
+// from h * vdim on, out_scale * weight * silu(gate) * o / rms(o) (the sum of squares in the order of the head norm's kernel);
+// else float, (o + D v) silu(gate).  TAPS 0: any number.
+template <int R4, bool DELTA, typename T, int TAPS>
 __global__ __launch_bounds__(DL_THREADS) void delta_step_kernel(T* __restrict__ out, int64_t out_stride, const ga_delta_args a,
                                                                 const float* __restrict__ weight, float eps, float out_scale) {
   constexpr int NB = 16 / R4;                              // column blocks that a wavefront has in registers at a time
+  constexpr int RD = 2;                                    // channels of a thread that are under way at a time
   __shared__ __attribute__((aligned(16))) float ks[64 * R4], qs[64 * R4];
   __shared__ float vs[DL_MAX_VDIM], os[DL_MAX_VDIM];
-  __shared__ float scratch[DL_WAVES], lengths[2];
+  __shared__ float lengths[2];
   const int e = blockIdx.x, h = blockIdx.y;
-  const int64_t t = a.cu[e];
-  if (a.cu[e + 1] - (int)t <= 0) return;
   const int tid = threadIdx.x, lane = tid % WAVE, wave = tid / WAVE, s = lane & 15;
-  const int per_group = a.heads / a.groups, g = h / per_group;
+  const int64_t t = a.cu[e];
   const int pos = a.q_start[e];
   const int64_t slot = a.slots[e];
+  if (a.cu[e + 1] - (int)t <= 0) return;
+  const int per_group = a.heads / a.groups, g = h / per_group;
   const int blocks = (a.vdim + 3) / 4;
+  const float* row = a.proj + t * a.stride;
+  // the channels first: they are what the rest waits for
+  const int total = 2 * a.dim + a.vdim;
+  auto channel = [&](int i) { return i < a.dim ? a.q_at + g * a.dim + i : i < 2 * a.dim ? a.k_at + g * a.dim + (i - a.dim) : a.v_at + h * a.vdim + (i - 2 * a.dim); };
+  constexpr int TP = TAPS ? TAPS : 1;
+  float own[RD], back[RD][TP], w[RD][TP], bias[RD];
+  auto ask = [&](int i0) {
+#pragma unroll
+    for (int r = 0; r < RD; ++r) {
+      const int i = i0 + r * DL_THREADS;
+      const int c = channel(i < total ? i : 0);
+      own[r] = row[a.conv_at + c];
+      bias[r] = a.conv_bias ? a.conv_bias[c] : 0.f;
+      if (TAPS) {
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) w[r][j] = a.conv_w[(int64_t)c * TAPS + j];
+#pragma unroll
+        for (int j = 0; j < TAPS - 1; ++j) {
+          const int p = pos - (TAPS - 1 - j);
+          back[r][j] = p >= 0 ? a.ring[(slot * TAPS + p % TP) * (int64_t)a.channels + c] : 0.f;
+        }
+      }
+    }
+  };
+  ask(tid);
+  const float za = row[a.a_at + h], zb = row[a.b_at + h], dt_bias = a.dt_bias[h], rate = a.rate[h];
+  float gate[2], wt[2];                                    // of the value columns tid and tid + DL_THREADS
+#pragma unroll
+  for (int r = 0; r < 2; ++r) {
+    const int i = tid + r * DL_THREADS;
+    gate[r] = i < a.vdim ? row[a.gate_at + h * a.vdim + i] : 0.f;
+    wt[r] = (DELTA && i < a.vdim) ? weight[i] : 0.f;
+  }
   float4* st = reinterpret_cast<float4*>(a.state) + (slot * a.heads + h) * blocks * (int64_t)(R4 * WAVE) + lane;
   float4 S[NB][R4];
   auto load = [&](int first) {
@@ -313,22 +385,34 @@ __global__ __launch_bounds__(DL_THREADS) void delta_step_kernel(T* __restrict__ 
     }
   };
   load(0);
-  const float2 c2 = dl_coefficients(a, t, h);
   for (int i = tid; i < 64 * R4; i += DL_THREADS)
     if (i >= a.dim) ks[i] = qs[i] = 0.f;
-  // the convolved channels: this head's values, its group's q and k
-  for (int i = tid; i < 2 * a.dim + a.vdim; i += DL_THREADS) {
-    const int c = i < a.dim ? a.q_at + g * a.dim + i : i < 2 * a.dim ? a.k_at + g * a.dim + (i - a.dim) : a.v_at + h * a.vdim + (i - 2 * a.dim);
-    const float own = a.proj[t * a.stride + a.conv_at + c];
-    const float* w = a.conv_w + (int64_t)c * a.taps;
-    float acc = a.conv_bias ? a.conv_bias[c] : 0.f;
-    for (int j = 0; j < a.taps - 1; ++j) acc = fmaf(w[j], dl_input(a, t, 0, pos, slot, a.taps - 1 - j, c), acc);
-    const float y = dl_silu(fmaf(w[a.taps - 1], own, acc));
-    if (a.taps > 1 && (i >= 2 * a.dim || h == g * per_group)) a.ring[(slot * a.taps + pos % a.taps) * (int64_t)a.channels + c] = own;
-    if (i < a.dim) qs[i] = y;
-    else if (i < 2 * a.dim) ks[i - a.dim] = y;
-    else vs[i - 2 * a.dim] = y;
+  for (int i0 = tid; i0 < total; i0 += RD * DL_THREADS) {
+    if (i0 != tid) ask(i0);
+#pragma unroll
+    for (int r = 0; r < RD; ++r) {
+      const int i = i0 + r * DL_THREADS;
+      if (i >= total) continue;
+      const int c = channel(i);
+      float acc = bias[r];
+      if (TAPS) {
+#pragma unroll
+        for (int j = 0; j < TAPS - 1; ++j) acc = fmaf(w[r][j], back[r][j], acc);
+        acc = fmaf(w[r][TP - 1], own[r], acc);
+      } else {
+        const float* wc = a.conv_w + (int64_t)c * a.taps;
+        for (int j = 0; j < a.taps - 1; ++j) acc = fmaf(wc[j], dl_input(a, t, 0, pos, slot, a.taps - 1 - j, c), acc);
+        acc = fmaf(wc[a.taps - 1], own[r], acc);
+      }
+      const float y = dl_silu(acc);
+      // the token's own row of the ring (the heads of a group share q and k: the first of them writes)
+      if (a.taps > 1 && (i >= 2 * a.dim || h == g * per_group)) a.ring[(slot * a.taps + pos % a.taps) * (int64_t)a.channels + c] = own[r];
+      if (i < a.dim) qs[i] = y;
+      else if (i < 2 * a.dim) ks[i - a.dim] = y;
+      else vs[i - 2 * a.dim] = y;
+    }
   }
+  const float2 c2 = dl_coefficients(DELTA, za, zb, dt_bias, rate);
   __syncthreads();
   if (DELTA) {
     if (wave < 2) {
@@ -363,17 +447,23 @@ __global__ __launch_bounds__(DL_THREADS) void delta_step_kernel(T* __restrict__ 
     }
   }
   __syncthreads();
-  const float* gate = a.proj + t * a.stride + a.gate_at + h * a.vdim;
   T* op = out + t * out_stride + (int64_t)h * a.vdim;
+  float rms = 1.f;
   if (DELTA) {
-    float ss = 0.f;
-    for (int i = tid; i < a.vdim; i += DL_THREADS) ss = fmaf(os[i], os[i], ss);
-    ss = block_sum<DL_WAVES>(ss, scratch);
-    const float rms = sqrtf(ss / (float)a.vdim + eps);
-    for (int i = tid; i < a.vdim; i += DL_THREADS) Num<T>::st(op + i, os[i] / rms * weight[i] * dl_silu(gate[i]) * out_scale);
-  } else {
-    const float skip = a.skip[h];
-    for (int i = tid; i < a.vdim; i += DL_THREADS) Num<T>::st(op + i, (os[i] + skip * vs[i]) * dl_silu(gate[i]));
+    float ss = 0.f;                                        // by every wavefront for itself
+    for (int i = 4 * lane; i < a.vdim; i += 4 * WAVE)
+#pragma unroll
+      for (int x = 0; x < 4; ++x)
+        if (i + x < a.vdim) ss = fmaf(os[i + x], os[i + x], ss);
+    rms = sqrtf(wave_sum(ss) / (float)a.vdim + eps);
+  }
+  const float skip = DELTA ? 0.f : a.skip[h];
+#pragma unroll
+  for (int r = 0; r < 2; ++r) {
+    const int i = tid + r * DL_THREADS;
+    if (i >= a.vdim) continue;
+    if (DELTA) Num<T>::st(op + i, os[i] / rms * wt[r] * dl_silu(gate[r]) * out_scale);
+    else Num<T>::st(op + i, (os[i] + skip * vs[i]) * dl_silu(gate[r]));
   }
 }
 
@@ -408,10 +498,14 @@ extern "C" int ga_delta_scan(void* out, const void* act, const ga_delta_args* ar
   const ga_delta_args& a = *args;
   const int rc = dl_check(a);
   if (rc) return rc;
-  dim3 grid(entries, a.heads, (a.vdim + DL_COLS - 1) / DL_COLS), block(DL_THREADS);
-#define GO(R4, D) hipLaunchKernelGGL((delta_scan_kernel<R4, D>), grid, block, 0, stream, (float*)out, (const float*)act, a)
-#define GR(D) do { const int r = (a.dim + 63) / 64; if (r == 1) GO(1, D); else if (r == 2) GO(2, D); else if (r == 3) GO(3, D); else GO(4, D); } while (0)
-  if (a.delta) GR(true); else GR(false);
+  // two column blocks to a wavefront, which read q and k from LDS once for both, where that still fills the chip
+  const int64_t wide = (int64_t)entries * a.heads * ((a.vdim + 2 * DL_COLS - 1) / (2 * DL_COLS));
+  const int cols = wide >= 384 ? 2 * DL_COLS : DL_COLS;
+  dim3 grid(entries, a.heads, (a.vdim + cols - 1) / cols), block(DL_THREADS);
+#define GO(R4, D, C) hipLaunchKernelGGL((delta_scan_kernel<R4, D, C>), grid, block, 0, stream, (float*)out, (const float*)act, a)
+#define GR(D, C) do { const int r = (a.dim + 63) / 64; if (r == 1) GO(1, D, C); else if (r == 2) GO(2, D, C); else if (r == 3) GO(3, D, C); else GO(4, D, C); } while (0)
+  if (cols > DL_COLS) { if (a.delta) GR(true, 2); else GR(false, 2); }
+  else { if (a.delta) GR(true, 1); else GR(false, 1); }
 #undef GR
 #undef GO
   return GA_CHECK_LAUNCH();
@@ -425,12 +519,14 @@ extern "C" int ga_delta_step(void* out, int64_t out_stride, const ga_delta_args*
   if (rc) return rc;
   if (a.delta ? !weight : out_bf16) return -6;
   dim3 grid(entries, a.heads), block(DL_THREADS);
-#define GO(R4, D, T) hipLaunchKernelGGL((delta_step_kernel<R4, D, T>), grid, block, 0, stream, (T*)out, out_stride, a, (const float*)weight, eps, out_scale)
+#define GT(R4, D, T, N) hipLaunchKernelGGL((delta_step_kernel<R4, D, T, N>), grid, block, 0, stream, (T*)out, out_stride, a, (const float*)weight, eps, out_scale)
+#define GO(R4, D, T) do { if (a.taps == 4) GT(R4, D, T, 4); else GT(R4, D, T, 0); } while (0)
 #define GR(D, T) do { const int r = (a.dim + 63) / 64; if (r == 1) GO(1, D, T); else if (r == 2) GO(2, D, T); else if (r == 3) GO(3, D, T); else GO(4, D, T); } while (0)
   if (!a.delta) GR(false, float);
   else if (out_bf16) GR(true, bf16_t);
   else GR(true, float);
 #undef GR
 #undef GO
+#undef GT
   return GA_CHECK_LAUNCH();
 }

@@ -210,12 +210,14 @@ int ga_attn_prefill(void* out, int64_t out_stride, const void* q, int64_t q_stri
 // * padded], k and v into their pages (k [pages, nkv, page_size, padded], v [pages, nkv, padded, page_size]), heads
 // padded with zeros; then (update_state) a second launch moves the state on by the step's tokens; proj may be float
 // beside a bfloat16 compute dtype (proj_bf16 0, is_bf16 1); stride: proj's row stride; head_eps >= 0: every head of q and k is
-// divided by its own root mean square and multiplied by gain float [2, hd] (q's, then k's)
+// divided by its own root mean square and multiplied by gain float [2, hd] (q's, then k's); bias: null, or one number per channel in the compute dtype, added to proj
+// (without a convolution and a norm over the whole projection)
 int ga_conv_rope_kv(void* q_out, const void* proj, const void* w, void* state, const void* slots, const void* token_entry,
                     const void* cu, const void* q_start, const void* positions, const void* cos_t, const void* sin_t,
                     const void* slot_mapping, void* k_pages, void* v_pages, int tokens, int entries, int nh, int nkv, int hd,
                     int vd, int padded, int rotary_dim, int taps, int page_size, int write_kv, int update_state, int is_bf16,
-                    int proj_bf16, void* row_scale, const void* gain, float norm_eps, int64_t stride, float head_eps, hipStream_t stream);
+                    int proj_bf16, void* row_scale, const void* gain, float norm_eps, int64_t stride, float head_eps,
+                    const void* bias, hipStream_t stream);
 
 // ---- output_norm.hip: residual[t] += scale * gain * y[t] / sqrt(mean(y[t]^2) + eps) (a norm on a sublayer's output, a
 // factor per channel behind it; gain and scale float [hidden], scale may be null); with `next` also next[t] = next_gain *

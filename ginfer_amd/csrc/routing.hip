@@ -70,6 +70,35 @@ __global__ __launch_bounds__(ROUTE_THREADS) void route_topk_kernel(const float* 
   }
 }
 
+// o[0 .. n) = w * row[0 .. n) by one wavefront (exact zeros where w is zero, whatever the row holds); four elements to an access, eight
+// accesses under way, where n and the addresses allow it
+__device__ __forceinline__ float4 router_load4(const float* p) { return *reinterpret_cast<const float4*>(p); }
+__device__ __forceinline__ float4 router_load4(const bf16_t* p) {
+  const uint2 u = *reinterpret_cast<const uint2*>(p);
+  return make_float4(__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u), __uint_as_float(u.y << 16),
+                     __uint_as_float(u.y & 0xffff0000u));
+}
+template <typename T>
+__device__ __forceinline__ void scaled_row(float* __restrict__ o, const T* __restrict__ row, float w, int n, int lane) {
+  if ((n & 3) == 0 && ((uintptr_t)o & 15) == 0 && ((uintptr_t)row & (4 * sizeof(T) - 1)) == 0) {
+    for (int i0 = 4 * lane; i0 < n; i0 += 8 * 4 * WAVE) {
+      float4 v[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const int i = i0 + u * 4 * WAVE;
+        v[u] = (w != 0.f && i < n) ? router_load4(row + i) : make_float4(0.f, 0.f, 0.f, 0.f);
+      }
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const int i = i0 + u * 4 * WAVE;
+        if (i < n) *reinterpret_cast<float4*>(o + i) = make_float4(w * v[u].x, w * v[u].y, w * v[u].z, w * v[u].w);
+      }
+    }
+  } else {
+    for (int i = lane; i < n; i += WAVE) o[i] = w == 0.f ? 0.f : w * Num<T>::ld(row + i);
+  }
+}
+
 // Routing by scores of every expert with a correction and groups of experts (one wavefront per token):
 //   s = sigmoid(z), or (softmax) the softmax of z over all experts;  c = s + correction (the choice score; without a correction c = s)
 //   the experts fall into `groups` equal groups of neighbours; a group's score is the sum of its `group_top` largest c; only
@@ -194,15 +223,13 @@ __global__ __launch_bounds__(ROUTE_THREADS) void route_groups_kernel(
     for (int k = 0; k < top; ++k) {
       if (chosen_i[k] < own) continue;
       const float w = plain[chosen_i[k]] * factor;
-      float* o = own_out + ((int64_t)k * gridDim.x + t) * hidden;
-      for (int i = lane; i < hidden; i += ROUTE_THREADS) o[i] = w * Num<T>::ld(row + i);
+      scaled_row(own_out + ((int64_t)k * gridDim.x + t) * hidden, row, w, hidden, lane);
     }
   } else {
     float w = 0.f;
     for (int k = 0; k < top; ++k)
       if (chosen_i[k] >= own) w += plain[chosen_i[k]] * factor;
-    float* o = own_out + t * hidden;
-    for (int i = lane; i < hidden; i += ROUTE_THREADS) o[i] = w == 0.f ? 0.f : w * Num<T>::ld(row + i);
+    scaled_row(own_out + t * hidden, row, w, hidden, lane);
   }
 }
 
@@ -260,13 +287,6 @@ __global__ __launch_bounds__(256) void weighted_silu_mul_kernel(T* __restrict__ 
   }
   if (V > 1) *reinterpret_cast<uint4*>(out + t * width + c) = res.u;
   else out[t * width + c] = res.e[0];
-}
-
-__device__ __forceinline__ float4 router_load4(const float* p) { return *reinterpret_cast<const float4*>(p); }
-__device__ __forceinline__ float4 router_load4(const bf16_t* p) {
-  const uint2 u = *reinterpret_cast<const uint2*>(p);
-  return make_float4(__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u), __uint_as_float(u.y << 16),
-                     __uint_as_float(u.y & 0xffff0000u));
 }
 
 // Router scores: z[t, e] = w[e] . x[t] + b[e] in 32-bit (x in the compute dtype or float, w and b float).  A wavefront per

@@ -1489,14 +1489,16 @@ def scaled_sum(a, b, sa, sb, dtype):
 
 
 def conv_rope_kv(proj, weight, state, slots, step, cos, sin, slot_mapping, k_pages, v_pages, num_heads, num_kv_heads, head_dim,
-                 value_dim, padded, dtype, write_kv=True, update_state=True, qk_gain=None, qk_eps=0.0, head_norm=False):
+                 value_dim, padded, dtype, write_kv=True, update_state=True, qk_gain=None, qk_eps=0.0, head_norm=False,
+                 bias=None):
     """Behind a fused q|k|v projection whose channels pass a short causal convolution: proj [T, (nh + nkv) hd + nkv vd] in
     the compute dtype `dtype` or in float32; weight float32 [channels, taps] (None: no convolution); state float32 [slots, taps - 1, channels]
     (None for one tap) and slots int64 [entries]; cos, sin float32 [positions, rotary_dim / 2] (None: no rotation).
     qk_gain float32 [(nh + nkv) hd] (no convolution then): q and k are divided by the root mean square of the token's WHOLE q
     (k) projection (eps qk_eps) and multiplied by the gain, before the rotation.
     head_norm: qk_gain is float32 [2, hd] instead, and every head of q and of k is divided by its own root mean square and
-    multiplied by its kind's gain.  proj's rows may be longer than its C columns (a view of a wider tensor).
+    multiplied by its kind's gain.  bias [C] in `dtype`: added to the projection (no convolution, no norm over the whole of it
+    then).  proj's rows may be longer than its C columns (a view of a wider tensor).
     Returns q [T, nh * padded], heads padded with zeros, and writes k and v (padded alike) into the pages at slot_mapping;
     moves the state on by the step's tokens."""
     _dev(proj, weight, state, slots, cos, sin, slot_mapping, k_pages, v_pages)
@@ -1533,6 +1535,10 @@ def conv_rope_kv(proj, weight, state, slots, step, cos, sin, slot_mapping, k_pag
               and slot_mapping.is_contiguous(), "slot_mapping must be contiguous int64 [T]")
         page_size = _check_pages(k_pages, v_pages, dtype, num_kv_heads, padded)
     _need(proj.dtype in (dtype, torch.float32), "proj must be %s or float32", dtype)
+    if bias is not None:
+        _dev(proj, bias)
+        _need(bias.dtype == dtype and bias.shape == (C,) and bias.is_contiguous() and weight is None and (qk_gain is None or head_norm),
+              "bias must be contiguous %s [%d], without a convolution and a norm over the whole projection", dtype, C)
     q = torch.empty((T, num_heads * padded), dtype=dtype, device=proj.device)
     row_scale = None
     if head_norm:
@@ -1550,7 +1556,7 @@ def conv_rope_kv(proj, weight, state, slots, step, cos, sin, slot_mapping, k_pag
                                _i(head_dim), _i(value_dim), _i(padded), _i(rotary_dim), _i(taps), _i(page_size),
                                _i(1 if write_kv else 0), _i(1 if update_state else 0), _i(_is_bf16(dtype)),
                                _i(_is_bf16(proj.dtype)), _ptr(row_scale), _ptr(qk_gain), _f(qk_eps),
-                               _i64(proj.stride(0)), _f(qk_eps if head_norm else -1.0), _stream()), "conv_rope_kv")
+                               _i64(proj.stride(0)), _f(qk_eps if head_norm else -1.0), _ptr(bias), _stream()), "conv_rope_kv")
     return q
 
 

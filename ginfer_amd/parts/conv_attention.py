@@ -136,10 +136,7 @@ class ConvAttention(Part):
         if self.learned_sink:
             self.sinks = t[n["sink"]].float().contiguous()
         if self.bias:
-            parts = [t[n[r] + "." + n["bias"]] for r in ("q", "k", "v")]
-            if self.head_gate:               # the gate's rows have none
-                parts.append(torch.zeros((self.nh,), dtype=parts[0].dtype, device=parts[0].device))
-            self.b_qkv = torch.cat(parts, dim=0).contiguous()
+            self.b_qkv = torch.cat([t[n[r] + "." + n["bias"]] for r in ("q", "k", "v")], dim=0).contiguous()
         if self.out_bias:
             self.b_o = t[n["o"] + "." + n["bias"]].contiguous()
         if self.head_norm_eps is not None:
@@ -159,16 +156,22 @@ class ConvAttention(Part):
     # (`ParallelSum`): the factor that it puts in front of the result rides on the gate.
     @property
     def shares_products(self):
-        return self.head_gate and self.b_o is None and not self.out_bias
+        return self.head_gate and not self.out_bias and (not self.bias or self._late_bias)
+
+    @property
+    def _late_bias(self):
+        """Whether the projection's bias is added behind the product, by the kernel that reads it: an addition of its own over
+        the product's rows is a pass over memory."""
+        return self.bias and not self.has_conv and self.qk_norm_eps is None
 
     @property
     def result_width(self):
         return self.nh * self.padded
 
     def hand_over_products(self):
-        """(the projection's matrix, its bias or None, the output's matrix): another part does both products from now on."""
-        out = (self.w_qkv, self.b_qkv, self.w_o)
-        self.w_qkv = self.b_qkv = self.w_o = None
+        """(the projection's matrix, the output's): another part does both products from now on, neither with a bias."""
+        out = (self.w_qkv, self.w_o)
+        self.w_qkv = self.w_o = None
         return out
 
     def core(self, proj, step, cache, out=None, out_scale=1.0):
@@ -180,11 +183,15 @@ class ConvAttention(Part):
                              None if state is None else state.slots, step, cos, sin, kv.slot_mapping, kv.k_pages, kv.v_pages,
                              self.nh, self.nkv, self.hd, self.vd, self.padded, self.dtype, write_kv=kv.owner,
                              update_state=state is not None and state.owner, qk_gain=self.qk_gain,
-                             qk_eps=self.qk_norm_eps or self.head_norm_eps or 0.0, head_norm=self.head_norm_eps is not None)
+                             qk_eps=self.qk_norm_eps or self.head_norm_eps or 0.0, head_norm=self.head_norm_eps is not None,
+                             bias=self.b_qkv if self._late_bias else None)
         return ops.paged_attention(q, kv.k_pages, kv.v_pages, kv.block_table, step, self.nh, self.nkv, self.padded,
                                    self.scale, self.window, sinks=self.sinks, chunk=self.chunk, soft_cap=self.soft_cap,
                                    gate=proj[:, self.width:] if self.head_gate else None, gate_scale=out_scale, out=out)
 
     def forward(self, x, step, cache):
-        a = self.core(linear(x, self.w_qkv, self.b_qkv, out_dtype=torch.float32), step, cache)
+        bias = None if self._late_bias or not self.bias else self.b_qkv
+        if bias is not None and self.head_gate:          # the gate's columns have none
+            bias = torch.cat([bias, torch.zeros((self.nh,), dtype=bias.dtype, device=bias.device)])
+        a = self.core(linear(x, self.w_qkv, bias, out_dtype=torch.float32), step, cache)
         return linear(a, self.w_o, self.b_o, parts_ok=self.b_o is None)

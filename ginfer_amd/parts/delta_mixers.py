@@ -49,7 +49,7 @@ class _DeltaMixer(Part):
         return self.nh * self.dv
 
     def hand_over_products(self):
-        out = (self.w_in, None, self.w_o)
+        out = (self.w_in, self.w_o)
         self.w_in = self.w_o = None
         return out
 

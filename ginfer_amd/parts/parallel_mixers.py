@@ -24,7 +24,7 @@ class ParallelSum(Part):
             raise ValueError("two mixers side by side, each with a name and a factor; got %d, %d, %d"
                              % (len(self.branches), len(self.names), len(self.scales)))
         self.dtype, self.device = dtype, device
-        self.w_in = self.b_in = self.w_out = None
+        self.w_in = self.w_out = None
         self.capturable = all(getattr(b, "capturable", False) for b in self.branches)
 
     def _shares(self):
@@ -53,17 +53,14 @@ class ParallelSum(Part):
     def _take_products(self):
         handed = [b.hand_over_products() for b in self.branches]
         self._columns, at = [], 0
-        for w_in, _, _ in handed:
+        for w_in, _ in handed:
             self._columns.append((at, at + w_in.shape[0]))
             at += w_in.shape[0]
         self.w_in = torch.cat([h[0] for h in handed], dim=0).contiguous()
-        if any(h[1] is not None for h in handed):
-            self.b_in = torch.cat([h[1] if h[1] is not None else torch.zeros(h[0].shape[:1], dtype=h[0].dtype, device=h[0].device)
-                                   for h in handed]).contiguous()
         widths = [b.result_width for b in self.branches]
         self._results = [(0, widths[0]), (widths[0], widths[0] + widths[1])]
         self._padding = -sum(widths) % 8             # the products take rows in steps of 8 elements
-        outs = [h[2] for h in handed]
+        outs = [h[1] for h in handed]
         if self._padding:
             outs.append(torch.zeros((outs[0].shape[0], self._padding), dtype=outs[0].dtype, device=outs[0].device))
         self.w_out = torch.cat(outs, dim=1).contiguous()
@@ -86,7 +83,7 @@ class ParallelSum(Part):
         return ops.scaled_sum(results[0], results[1], self.scales[0], self.scales[1], self.dtype)
 
     def _forward_shared(self, x, step, cache):
-        proj = linear(x, self.w_in, self.b_in, out_dtype=torch.float32)
+        proj = linear(x, self.w_in, None, out_dtype=torch.float32)
         make = torch.zeros if self._padding else torch.empty
         both = make((x.shape[0], self.w_out.shape[1]), dtype=self.dtype, device=x.device)
         at = 0
