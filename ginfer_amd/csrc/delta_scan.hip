@@ -5,9 +5,10 @@
 //   both         a = exp(-rate * softplus(za + bias))
 // q, k and v are columns of one 32-bit projection that have passed a short causal convolution over time (per channel) and silu;
 // za, zb and the gate z of the output are columns of the same projection.
-//   prepare   a step's convolved channels [tokens, channels] (float): a thread a channel and 8 tokens, unit vectors made in LDS
-//   scan      any entries: a workgroup owns (entry, head, 16 value columns) and walks the entry's tokens 16 at a time, their q,
-//             k and v in LDS, asked for a tile ahead.  16 lanes of a wavefront share a column: lane s keeps rows 64 j + 4 s .. + 3
+//   prepare   a step's convolved channels (float): a thread a channel and 8 tokens, unit vectors made in LDS; and the decays and
+//             steps of its tokens.  A row holds q and k, 64-aligned heads (`pad` wide), then v: what a tile of the scan loads
+//   scan      any entries: a workgroup owns (entry, head, 16 or 32 value columns) and walks the entry's tokens 16 at a time,
+//             their q, k and v in LDS, asked for from memory two tiles ahead and stored one ahead, one barrier a tile.  16 lanes of a wavefront share a column: lane s keeps rows 64 j + 4 s .. + 3
 //             of it in registers, and their sums meet in four rotations inside the 16 lanes
 //   step      single tokens, all in one launch: a workgroup owns (entry, head), makes its channels, moves the state (all of
 //             its loads under way before the channels are made) and, for the delta rule, norms and gates the head's result
@@ -20,7 +21,6 @@
 
 #define DL_THREADS 256
 #define DL_WAVES (DL_THREADS / WAVE)
-#define DL_TILE 16           // tokens per trip through LDS
 #define DL_COLS 16           // value columns of a workgroup of the scan: four to a wavefront
 #define DL_MAX_TAPS 16
 #define DL_MAX_VDIM 512
@@ -62,7 +62,7 @@ __device__ __forceinline__ float dl_inverse_length(const float* x, int n, float 
   return 1.f / sqrtf(wave_sum(ss) + eps);
 }
 
-// A token's share of one column in a lane: rows 64 j + 4 s .. + 3
+// A token's share of one column in a lane: rows 64 j + 4 s .. + 3.  Returns the lane's part of o, for dl_row_sum
 template <int R4, bool DELTA>
 __device__ __forceinline__ float dl_advance(float4 (&S)[R4], const float4 (&k)[R4], const float4 (&q)[R4], float v, float a, float b) {
   float u;
@@ -91,13 +91,31 @@ __device__ __forceinline__ float dl_advance(float4 (&S)[R4], const float4 (&k)[R
     o0 = fmaf(S[j].z, q[j].z, o0);
     o1 = fmaf(S[j].w, q[j].w, o1);
   }
-  return dl_row_sum(o0 + o1);
+  return o0 + o1;
 }
 
 // ---------------------------------------------------------------------------------------------------- prepare
-// grid (token tiles, channel blocks): first the blocks of whole q and k heads (DL_THREADS / dim heads each), then the others
+// A prepared row: q [groups][pad], k [groups][pad], v [heads * vdim], rounded up to 4; pad = dim rounded up to 64 (what lies between
+// dim and pad is not written and not used).
+__host__ __device__ __forceinline__ int dl_pad(const ga_delta_args& a) { return (a.dim + 63) / 64 * 64; }
+__host__ __device__ __forceinline__ int64_t dl_row(const ga_delta_args& a) {
+  return ((int64_t)2 * a.groups * dl_pad(a) + (int64_t)a.heads * a.vdim + 3) / 4 * 4;
+}
+// where convolved channel c lies in a prepared row
+__device__ __forceinline__ int dl_place(const ga_delta_args& a, int c) {
+  const int n = a.groups * a.dim, pad = dl_pad(a);
+  int i = c - a.q_at;
+  if (i >= 0 && i < n) return i / a.dim * pad + i % a.dim;
+  i = c - a.k_at;
+  if (i >= 0 && i < n) return (a.groups + i / a.dim) * pad + i % a.dim;
+  return 2 * a.groups * pad + (c - a.v_at);
+}
+
+// grid (token tiles, channel blocks): first the blocks of whole q and k heads (DL_THREADS / dim heads each), then the others, and
+// the last for the decays and steps: coef float2 [tokens][heads]
 template <int TAPS, int TB>      // TAPS 0: any number
-__global__ __launch_bounds__(DL_THREADS) void delta_prepare_kernel(float* __restrict__ out, const ga_delta_args a,
+__global__ __launch_bounds__(DL_THREADS) void delta_prepare_kernel(float* __restrict__ out, float2* __restrict__ coef,
+                                                                   const ga_delta_args a,
                                                                    const int32_t* __restrict__ token_entry, int tokens) {
   __shared__ float ys[TB][DL_THREADS];
   __shared__ float factor[TB][DL_THREADS];
@@ -117,6 +135,17 @@ __global__ __launch_bounds__(DL_THREADS) void delta_prepare_kernel(float* __rest
   const bool live = c < last;
   const int64_t t0 = (int64_t)blockIdx.x * TB;
   const int nt = min((int64_t)TB, tokens - t0);
+  if (blockIdx.y == gridDim.y - 1) {
+    for (int i = tid; i < nt * a.heads; i += DL_THREADS) {
+      const int64_t t = t0 + i / a.heads;
+      const int h = i % a.heads;
+      const float* row = a.proj + t * a.stride;
+      coef[t * a.heads + h] = dl_coefficients(a.delta, row[a.a_at + h], row[a.b_at + h], a.dt_bias[h], a.rate[h]);
+    }
+    return;
+  }
+  float* to = out + t0 * dl_row(a) + (live ? dl_place(a, c) : 0);
+  const int64_t to_row = dl_row(a);
   float y[TB];
 #pragma unroll
   for (int i = 0; i < TB; ++i) y[i] = 0.f;
@@ -167,7 +196,7 @@ __global__ __launch_bounds__(DL_THREADS) void delta_prepare_kernel(float* __rest
     if (live) {
 #pragma unroll
       for (int i = 0; i < TB; ++i)
-        if (i < nt) out[(t0 + i) * a.channels + c] = y[i];
+        if (i < nt) to[i * to_row] = y[i];
     }
     return;
   }
@@ -185,20 +214,23 @@ __global__ __launch_bounds__(DL_THREADS) void delta_prepare_kernel(float* __rest
     const int hh = tid / a.dim;
 #pragma unroll
     for (int i = 0; i < TB; ++i)
-      if (i < nt) out[(t0 + i) * a.channels + c] = y[i] * factor[i][hh] * scale;
+      if (i < nt) to[i * to_row] = y[i] * factor[i][hh] * scale;
   }
 }
 
 // ---------------------------------------------------------------------------------------------------- scan
-// grid (entries, heads, blocks of 16 C value columns): C blocks of four columns to a wavefront.  act: the prepared channels
-// [tokens, channels].  out float [tokens, heads, vdim]: o, or for the state space (o + D v) silu(z).
-template <int R4, bool DELTA, int C>
-__global__ __launch_bounds__(DL_THREADS) void delta_scan_kernel(float* __restrict__ out, const float* __restrict__ act,
-                                                                const ga_delta_args a) {
+// grid (entries, heads, blocks of 16 C value columns): C blocks of four columns to a wavefront; TILE tokens (8 or 16) per trip
+// through LDS.  act, coef: as prepare leaves them.  out float [tokens, heads, vdim]: o, or for the state space (o + D v) silu(z).
+template <int R4, bool DELTA, int C, int TILE>
+__global__ __launch_bounds__(DL_THREADS) __attribute__((amdgpu_waves_per_eu(1, 4))) void delta_scan_kernel(
+    float* __restrict__ out, const float* __restrict__ act, const float2* __restrict__ coef, const ga_delta_args a) {
   constexpr int DP = 64 * R4, COLS = DL_COLS * C;
-  __shared__ __attribute__((aligned(16))) float ks[DL_TILE][DP], qs[DL_TILE][DP];
-  __shared__ float vs[DL_TILE][COLS], os[DL_TILE][COLS + 1];
-  __shared__ float2 cf[DL_TILE];
+  constexpr int QUADS = TILE * DP / 4 / DL_THREADS;          // 16-byte pieces of a tile's q (and of its k) that a thread brings
+  constexpr int VALS = TILE * COLS / DL_THREADS > 0 ? TILE * COLS / DL_THREADS : 1;
+  static_assert(TILE * DP % (4 * DL_THREADS) == 0, "whole pieces");
+  __shared__ __attribute__((aligned(16))) float ks[2][TILE][DP], qs[2][TILE][DP];
+  __shared__ float vs[2][TILE][COLS];
+  __shared__ float2 cf[2][TILE];
   const int e = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * COLS;
   const int first = a.cu[e], n = a.cu[e + 1] - first;
   if (n <= 0) return;
@@ -214,96 +246,129 @@ __global__ __launch_bounds__(DL_THREADS) void delta_scan_kernel(float* __restric
 #pragma unroll
     for (int j = 0; j < R4; ++j)
       S[c][j] = (start > 0 && cb + c < blocks) ? st[(c * R4 + j) * WAVE] : make_float4(0.f, 0.f, 0.f, 0.f);
-  constexpr int PER = DL_TILE * DP / DL_THREADS;
-  float rq[PER], rk[PER], rv[C], rz[C], ra = 0.f, rb = 0.f;
-#pragma unroll
-  for (int c = 0; c < C; ++c) rz[c] = 0.f;
-  const float* qp = act + a.q_at + g * a.dim;
-  const float* kp = act + a.k_at + g * a.dim;
-  const float* vp = act + a.v_at + h * a.vdim + v0;
-  // this thread's places in a tile of values and results: (row ft[c], column fc[c])
-  auto ft = [&](int c) { return (tid + c * DL_THREADS) / COLS; };
-  auto fc = [&](int c) { return (tid + c * DL_THREADS) % COLS; };
-  // everything of a tile is only asked for here: nothing uses what a load brings before the tile is stored
+  const int row = (int)dl_row(a);
+  const float* qp = act + (int64_t)first * row + g * DP;
+  const float* kp = qp + a.groups * DP;
+  const float* vp = act + (int64_t)first * row + 2 * a.groups * DP + h * a.vdim + v0;
+  const float* zp = a.proj + (int64_t)first * a.stride + a.gate_at + h * a.vdim + v0;
+  const float2* cp = coef + (int64_t)first * a.heads + h;
+  float* op = out + ((int64_t)first * a.heads + h) * a.vdim + v0;
+  float4 rq[QUADS], rk[QUADS];
+  float rv[VALS];
+  float2 rc;
+  // a tile's operands: only asked for here.  Rows behind the entry's last are read as the last and never used; so are columns.
   auto fetch = [&](int t0) {
-    const int nt = min(DL_TILE, n - t0);
+    const int nt = min(TILE, n - t0);
+    const float* q = qp + (int64_t)t0 * row;
+    const float* k = kp + (int64_t)t0 * row;
+    const float* v = vp + (int64_t)t0 * row;
 #pragma unroll
-    for (int x = 0; x < PER; ++x) {
-      const int idx = tid + x * DL_THREADS, tt = idx / DP, i = idx % DP;
-      const bool in = tt < nt && i < a.dim;
-      const int64_t at = (int64_t)(first + t0 + tt) * a.channels + i;
-      rq[x] = in ? qp[at] : 0.f;
-      rk[x] = in ? kp[at] : 0.f;
-    }
-#pragma unroll
-    for (int c = 0; c < C; ++c) {
-      const bool in = ft(c) < nt && v0 + fc(c) < a.vdim;
-      const int64_t row = first + t0 + ft(c);
-      rv[c] = in ? vp[row * a.channels + fc(c)] : 0.f;
-      if (!DELTA) rz[c] = in ? a.proj[row * a.stride + a.gate_at + h * a.vdim + v0 + fc(c)] : 0.f;
-    }
-    if (tid < nt) {
-      const float* row = a.proj + (int64_t)(first + t0 + tid) * a.stride;
-      ra = row[a.a_at + h];
-      rb = row[a.b_at + h];
-    }
-  };
-  const float skip = DELTA ? 0.f : a.skip[h], dt_bias = a.dt_bias[h], rate = a.rate[h];
-  fetch(0);
-  for (int t0 = 0; t0 < n; t0 += DL_TILE) {
-    const int nt = min(DL_TILE, n - t0);
-    __syncthreads();                                       // the tile before is read out
-#pragma unroll
-    for (int x = 0; x < PER; ++x) {
+    for (int x = 0; x < QUADS; ++x) {
       const int idx = tid + x * DL_THREADS;
-      qs[idx / DP][idx % DP] = rq[x];
-      ks[idx / DP][idx % DP] = rk[x];
+      const int at = min(idx / (DP / 4), nt - 1) * row + 4 * (idx % (DP / 4));
+      rq[x] = *reinterpret_cast<const float4*>(q + at);
+      rk[x] = *reinterpret_cast<const float4*>(k + at);
     }
-    float z[C], v_own[C];
+#pragma unroll
+    for (int x = 0; x < VALS; ++x) {
+      const int idx = tid + x * DL_THREADS;
+      rv[x] = v[min(idx / COLS, nt - 1) * row + min(idx % COLS, a.vdim - 1 - v0)];
+    }
+    rc = cp[(int64_t)(t0 + min(tid, nt - 1)) * a.heads];
+  };
+  const bool ragged = a.dim != DP;                           // the rows beyond dim are zeros
+  auto store = [&](int b) {
+#pragma unroll
+    for (int x = 0; x < QUADS; ++x) {
+      const int idx = tid + x * DL_THREADS, tt = idx / (DP / 4), i = 4 * (idx % (DP / 4));
+      float4 q = rq[x], k = rk[x];
+      if (ragged) {
+        q = make_float4(i < a.dim ? q.x : 0.f, i + 1 < a.dim ? q.y : 0.f, i + 2 < a.dim ? q.z : 0.f, i + 3 < a.dim ? q.w : 0.f);
+        k = make_float4(i < a.dim ? k.x : 0.f, i + 1 < a.dim ? k.y : 0.f, i + 2 < a.dim ? k.z : 0.f, i + 3 < a.dim ? k.w : 0.f);
+      }
+      *reinterpret_cast<float4*>(&qs[b][tt][i]) = q;
+      *reinterpret_cast<float4*>(&ks[b][tt][i]) = k;
+    }
+#pragma unroll
+    for (int x = 0; x < VALS; ++x) {
+      const int idx = tid + x * DL_THREADS;
+      if (idx < TILE * COLS) vs[b][idx / COLS][idx % COLS] = rv[x];
+    }
+    if (tid < TILE) cf[b][tid] = rc;
+  };
+  const float skip = DELTA ? 0.f : a.skip[h];
+  fetch(0);
+  store(0);
+  if (TILE < n) fetch(TILE);
+  __syncthreads();
+  int b = 0;
+  for (int t0 = 0; t0 < n; t0 += TILE, b ^= 1) {
+    const int nt = min(TILE, n - t0);
+    // lane s of a column keeps token s's result (and its gate): no branch stands between the tokens
+    float mine[C], z[C];
 #pragma unroll
     for (int c = 0; c < C; ++c) {
-      vs[ft(c)][fc(c)] = rv[c];
-      z[c] = rz[c];
-      v_own[c] = rv[c];
+      mine[c] = 0.f;
+      z[c] = (!DELTA && s < nt && col + 4 * c < a.vdim - v0) ? zp[(int64_t)(t0 + s) * a.stride + col + 4 * c] : 0.f;
     }
-    if (tid < DL_TILE) cf[tid] = dl_coefficients(DELTA, ra, rb, dt_bias, rate);
-    __syncthreads();
-    if (t0 + DL_TILE < n) fetch(t0 + DL_TILE);
-    // lane s of a column keeps token s's result: no branch stands between the tokens
-    float mine[C];
-#pragma unroll
-    for (int c = 0; c < C; ++c) mine[c] = 0.f;
-    auto token = [&](int tt) {
-      float4 k[R4], q[R4];
+    struct Token { float4 k[R4], q[R4]; float2 ab; float v[C]; };
+    auto read = [&](int tt, Token& x) {
 #pragma unroll
       for (int j = 0; j < R4; ++j) {
-        k[j] = *reinterpret_cast<const float4*>(&ks[tt][64 * j + 4 * s]);
-        q[j] = *reinterpret_cast<const float4*>(&qs[tt][64 * j + 4 * s]);
+        x.k[j] = *reinterpret_cast<const float4*>(&ks[b][tt][64 * j + 4 * s]);
+        x.q[j] = *reinterpret_cast<const float4*>(&qs[b][tt][64 * j + 4 * s]);
       }
-      const float2 ab = cf[tt];
+      x.ab = cf[b][tt];
+#pragma unroll
+      for (int c = 0; c < C; ++c) x.v[c] = vs[b][tt][col + 4 * c];
+    };
+    auto keep = [&](int tt, const float (&part)[C]) {
 #pragma unroll
       for (int c = 0; c < C; ++c) {
-        const float o = dl_advance<R4, DELTA>(S[c], k, q, vs[tt][col + 4 * c], ab.x, ab.y);
+        const float o = dl_row_sum(part[c]);
         mine[c] = s == tt ? o : mine[c];
       }
     };
-    if (nt == DL_TILE) {
+    if (nt == TILE) {
+      // a token's operands are read while the one before is worked on (its reads may not sink below this line), and the sum of a
+      // result fills the waits of the next token's chain
+      Token x[2];
+      float part[2][C];
+      read(0, x[0]);
 #pragma unroll
-      for (int tt = 0; tt < DL_TILE; ++tt) token(tt);
+      for (int tt = 0; tt < TILE; ++tt) {
+        if (tt + 1 < TILE) read(tt + 1, x[(tt + 1) & 1]);
+        __builtin_amdgcn_sched_barrier(0);
+        const Token& y = x[tt & 1];
+#pragma unroll
+        for (int c = 0; c < C; ++c) part[tt & 1][c] = dl_advance<R4, DELTA>(S[c], y.k, y.q, y.v[c], y.ab.x, y.ab.y);
+        if (tt > 0) keep(tt - 1, part[(tt - 1) & 1]);
+      }
+      keep(TILE - 1, part[(TILE - 1) & 1]);
     } else {
-      for (int tt = 0; tt < nt; ++tt) token(tt);
-    }
+      for (int tt = 0; tt < nt; ++tt) {
+        Token y;
+        read(tt, y);
+        float part[C];
 #pragma unroll
-    for (int c = 0; c < C; ++c) os[s][col + 4 * c] = mine[c];
-    __syncthreads();
-#pragma unroll
-    for (int c = 0; c < C; ++c) {
-      if (ft(c) < nt && v0 + fc(c) < a.vdim) {
-        float o = os[ft(c)][fc(c)];
-        if (!DELTA) o = (o + skip * v_own[c]) * dl_silu(z[c]);
-        out[((int64_t)(first + t0 + ft(c)) * a.heads + h) * a.vdim + v0 + fc(c)] = o;
+        for (int c = 0; c < C; ++c) part[c] = dl_advance<R4, DELTA>(S[c], y.k, y.q, y.v[c], y.ab.x, y.ab.y);
+        keep(tt, part);
       }
     }
+    if (s < nt) {
+#pragma unroll
+      for (int c = 0; c < C; ++c)
+        if (col + 4 * c < a.vdim - v0) {
+          float o = mine[c];
+          if (!DELTA) o = (o + skip * vs[b][s][col + 4 * c]) * dl_silu(z[c]);
+          op[(int64_t)(t0 + s) * a.heads * a.vdim + col + 4 * c] = o;
+        }
+    }
+    if (t0 + TILE < n) {
+      store(b ^ 1);
+      if (t0 + 2 * TILE < n) fetch(t0 + 2 * TILE);
+    }
+    __syncthreads();
   }
 #pragma unroll
   for (int c = 0; c < C; ++c)
@@ -439,7 +504,7 @@ __global__ __launch_bounds__(DL_THREADS) void delta_step_kernel(T* __restrict__ 
       const int cb = first + b * DL_WAVES + wave;
       if (cb < blocks) {
         const int col = cb * 4 + (lane >> 4);
-        const float o = dl_advance<R4, DELTA>(S[b], k, q, col < a.vdim ? vs[col] : 0.f, c2.x, c2.y);
+        const float o = dl_row_sum(dl_advance<R4, DELTA>(S[b], k, q, col < a.vdim ? vs[col] : 0.f, c2.x, c2.y));
 #pragma unroll
         for (int j = 0; j < R4; ++j) st[(int64_t)cb * (R4 * WAVE) + j * WAVE] = S[b][j];
         if (s == 0 && col < a.vdim) os[col] = o;
@@ -475,17 +540,19 @@ static int dl_check(const ga_delta_args& a) {
   return 0;
 }
 
-extern "C" int ga_delta_prepare(void* act, const ga_delta_args* args, const void* token_entry, int tokens, hipStream_t stream) {
+extern "C" int64_t ga_delta_row(const ga_delta_args* args) { return dl_row(*args); }
+
+extern "C" int ga_delta_prepare(void* act, void* coef, const ga_delta_args* args, const void* token_entry, int tokens, hipStream_t stream) {
   if (tokens <= 0) return 0;
   const ga_delta_args& a = *args;
   const int rc = dl_check(a);
   if (rc) return rc;
   const int units = a.delta ? 2 * a.groups : 0, heads_here = a.delta ? DL_THREADS / a.dim : 1;
   const int plain = a.channels - units * a.dim;
-  const int64_t blocks = (units + heads_here - 1) / heads_here + (plain + DL_THREADS - 1) / DL_THREADS;
-  if (plain < 0 || blocks > 65535) return -5;
+  const int64_t blocks = (units + heads_here - 1) / heads_here + (plain + DL_THREADS - 1) / DL_THREADS + 1;
+  if (plain < 0 || blocks > 65535 || dl_row(a) > (1 << 26)) return -5;
 #define GO(TAPS, TB) hipLaunchKernelGGL((delta_prepare_kernel<TAPS, TB>), dim3((tokens + TB - 1) / TB, (unsigned)blocks), dim3(DL_THREADS), 0, \
-                                        stream, (float*)act, a, (const int32_t*)token_entry, tokens)
+                                        stream, (float*)act, (float2*)coef, a, (const int32_t*)token_entry, tokens)
   const bool few = (int64_t)tokens * blocks <= 2048;         // a token to a workgroup while that does not fill the chip
   if (a.taps == 4) { if (few) GO(4, 1); else GO(4, DL_PREP_TOKENS); }
   else { if (few) GO(0, 1); else GO(0, DL_PREP_TOKENS); }
@@ -493,7 +560,7 @@ extern "C" int ga_delta_prepare(void* act, const ga_delta_args* args, const void
   return GA_CHECK_LAUNCH();
 }
 
-extern "C" int ga_delta_scan(void* out, const void* act, const ga_delta_args* args, int entries, hipStream_t stream) {
+extern "C" int ga_delta_scan(void* out, const void* act, const void* coef, const ga_delta_args* args, int entries, hipStream_t stream) {
   if (entries <= 0) return 0;
   const ga_delta_args& a = *args;
   const int rc = dl_check(a);
@@ -502,8 +569,10 @@ extern "C" int ga_delta_scan(void* out, const void* act, const ga_delta_args* ar
   const int64_t wide = (int64_t)entries * a.heads * ((a.vdim + 2 * DL_COLS - 1) / (2 * DL_COLS));
   const int cols = wide >= 384 ? 2 * DL_COLS : DL_COLS;
   dim3 grid(entries, a.heads, (a.vdim + cols - 1) / cols), block(DL_THREADS);
-#define GO(R4, D, C) hipLaunchKernelGGL((delta_scan_kernel<R4, D, C>), grid, block, 0, stream, (float*)out, (const float*)act, a)
-#define GR(D, C) do { const int r = (a.dim + 63) / 64; if (r == 1) GO(1, D, C); else if (r == 2) GO(2, D, C); else if (r == 3) GO(3, D, C); else GO(4, D, C); } while (0)
+  if (((uintptr_t)act & 15) || dl_row(a) > (1 << 26)) return -5;
+#define GO(R4, D, C, TILE) hipLaunchKernelGGL((delta_scan_kernel<R4, D, C, TILE>), grid, block, 0, stream, (float*)out, (const float*)act, (const float2*)coef, a)
+  // (the widest keys take half the tokens a trip: two buffers of 16 would not fit the LDS)
+#define GR(D, C) do { const int r = (a.dim + 63) / 64; if (r == 1) GO(1, D, C, 16); else if (r == 2) GO(2, D, C, 16); else if (r == 3) GO(3, D, C, 16); else GO(4, D, C, 8); } while (0)
   if (cols > DL_COLS) { if (a.delta) GR(true, 2); else GR(false, 2); }
   else { if (a.delta) GR(true, 1); else GR(false, 1); }
 #undef GR

@@ -338,10 +338,12 @@ typedef struct {
   int channels, taps, heads, groups, dim, vdim, delta;
   float q_scale, unit_eps;
 } ga_delta_args;
-// act float [tokens, channels]: convolved, silu, q and k (delta) as unit vectors, q times q_scale
-int ga_delta_prepare(void* act, const ga_delta_args* args, const void* token_entry, int tokens, hipStream_t stream);
+// act float [tokens, ga_delta_row(args)]: the channels convolved, silu, q and k (delta) as unit vectors, q times q_scale, as the
+// scan reads them (16-byte aligned); coef float [tokens, heads, 2]: decays and steps
+int64_t ga_delta_row(const ga_delta_args* args);
+int ga_delta_prepare(void* act, void* coef, const ga_delta_args* args, const void* token_entry, int tokens, hipStream_t stream);
 // out float [tokens, heads, vdim]: o (delta), or (o + skip v) silu(gate); advances state and ring
-int ga_delta_scan(void* out, const void* act, const ga_delta_args* args, int entries, hipStream_t stream);
+int ga_delta_scan(void* out, const void* act, const void* coef, const ga_delta_args* args, int entries, hipStream_t stream);
 // every entry brings one token: all of it in one launch; delta: out (compute dtype, row stride out_stride) = out_scale * weight *
 // silu(gate) * o / rms(o), else float, as the scan's
 int ga_delta_step(void* out, int64_t out_stride, const ga_delta_args* args, const void* weight, float eps, float out_scale,

@@ -1755,10 +1755,12 @@ def delta_recurrence(proj, conv_weight, conv_bias, rate, dt_bias, skip, ring, st
         _check(lib.ga_delta_step(_ptr(o), _i64(o.stride(0)), ctypes.byref(args), _ptr(weight), _f(eps), _f(out_scale),
                                  _i(_is_bf16(dtype) if delta else 0), _i(E), _stream()), "delta_step")
         return o
-    act = torch.empty((T, C), dtype=torch.float32, device=proj.device)
+    lib.ga_delta_row.restype = ctypes.c_int64
+    act = torch.empty((T, lib.ga_delta_row(ctypes.byref(args))), dtype=torch.float32, device=proj.device)
+    coef = torch.empty((T, heads, 2), dtype=torch.float32, device=proj.device)
     o = torch.empty((T, heads, vdim), dtype=torch.float32, device=proj.device)
-    _check(lib.ga_delta_prepare(_ptr(act), ctypes.byref(args), _ptr(step.token_entry), _i(T), _stream()), "delta_prepare")
-    _check(lib.ga_delta_scan(_ptr(o), _ptr(act), ctypes.byref(args), _i(E), _stream()), "delta_scan")
+    _check(lib.ga_delta_prepare(_ptr(act), _ptr(coef), ctypes.byref(args), _ptr(step.token_entry), _i(T), _stream()), "delta_prepare")
+    _check(lib.ga_delta_scan(_ptr(o), _ptr(act), _ptr(coef), ctypes.byref(args), _i(E), _stream()), "delta_scan")
     if not delta:
         return o
     return head_norm_gate(o, weight, eps, dtype, proj=proj, gate_start=at["gate"], out=out, out_scale=out_scale)
