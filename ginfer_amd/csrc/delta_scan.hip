@@ -10,24 +10,14 @@
 //   scan      any entries: a workgroup owns (entry, head, 16 or 32 value columns) and walks the entry's tokens 16 at a time,
 //             their q, k and v in LDS, asked for from memory two tiles ahead and stored one ahead, one barrier a tile.  16 lanes of a wavefront share a column: lane s keeps rows 64 j + 4 s .. + 3
 //             of it in registers, and their sums meet in four rotations inside the 16 lanes
+//             (delta_chunk.hip does the same in chunks on the matrix cores, where results may differ by rounding with the cut)
 //   step      single tokens, all in one launch: a workgroup owns (entry, head), makes its channels, moves the state (all of
 //             its loads under way before the channels are made) and, for the delta rule, norms and gates the head's result
 // The sums of a token are taken in the same order in scan and step, so results do not depend on how the tokens were cut.
 // State layouts.  S: [slot][head][vdim / 4][dim / 64][lane][4], the order in which a wavefront reads it (rows beyond dim hold
 // zeros).  The convolution's inputs: a ring [slot][taps][channels], the row p % taps being position p's: a step's own row is
 // none of the taps - 1 rows it reads, so a workgroup may write it while another one still reads.
-#include "common.h"
-#include "ginfer_amd.h"
-
-#define DL_THREADS 256
-#define DL_WAVES (DL_THREADS / WAVE)
-#define DL_COLS 16           // value columns of a workgroup of the scan: four to a wavefront
-#define DL_MAX_TAPS 16
-#define DL_MAX_VDIM 512
-#define DL_PREP_TOKENS 8
-
-__device__ __forceinline__ float dl_silu(float z) { return z / (1.f + expf(-z)); }
-__device__ __forceinline__ float dl_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+#include "delta_common.h"
 
 // the sum over the 16 lanes of a row, the same bits in every lane: rotations by 8, 4, 2 and 1
 template <int CTRL>
@@ -40,19 +30,6 @@ __device__ __forceinline__ float dl_row_sum(float v) {
   v += dl_rotated<0x122>(v);
   v += dl_rotated<0x121>(v);
   return v;
-}
-
-// The input of channel c at `back` tokens before the token at row t (place `local` of its entry's tokens, position pos)
-__device__ __forceinline__ float dl_input(const ga_delta_args& a, int64_t t, int local, int pos, int64_t slot, int back, int c) {
-  if (local >= back) return a.proj[(t - back) * a.stride + a.conv_at + c];
-  if (pos < back) return 0.f;
-  return a.ring[(slot * a.taps + (pos - back) % a.taps) * (int64_t)a.channels + c];
-}
-
-// decay and step of a head from its two columns of the projection
-__device__ __forceinline__ float2 dl_coefficients(bool delta, float za, float zb, float dt_bias, float rate) {
-  const float sp = dl_softplus(za + dt_bias);
-  return make_float2(expf(-rate * sp), delta ? 1.f / (1.f + expf(-zb)) : sp);
 }
 
 // 1 / the length of x[0 .. n) (n elements in LDS), by one wavefront
@@ -95,28 +72,12 @@ __device__ __forceinline__ float dl_advance(float4 (&S)[R4], const float4 (&k)[R
 }
 
 // ---------------------------------------------------------------------------------------------------- prepare
-// A prepared row: q [groups][pad], k [groups][pad], v [heads * vdim], rounded up to 4; pad = dim rounded up to 64 (what lies between
-// dim and pad is not written and not used).
-__host__ __device__ __forceinline__ int dl_pad(const ga_delta_args& a) { return (a.dim + 63) / 64 * 64; }
-__host__ __device__ __forceinline__ int64_t dl_row(const ga_delta_args& a) {
-  return ((int64_t)2 * a.groups * dl_pad(a) + (int64_t)a.heads * a.vdim + 3) / 4 * 4;
-}
-// where convolved channel c lies in a prepared row
-__device__ __forceinline__ int dl_place(const ga_delta_args& a, int c) {
-  const int n = a.groups * a.dim, pad = dl_pad(a);
-  int i = c - a.q_at;
-  if (i >= 0 && i < n) return i / a.dim * pad + i % a.dim;
-  i = c - a.k_at;
-  if (i >= 0 && i < n) return (a.groups + i / a.dim) * pad + i % a.dim;
-  return 2 * a.groups * pad + (c - a.v_at);
-}
-
 // grid (token tiles, channel blocks): first the blocks of whole q and k heads (DL_THREADS / dim heads each), then the others, and
-// the last for the decays and steps: coef float2 [tokens][heads]
+// the last for the decays (logs: their logarithms) and steps: coef float2 [tokens][heads]
 template <int TAPS, int TB>      // TAPS 0: any number
 __global__ __launch_bounds__(DL_THREADS) void delta_prepare_kernel(float* __restrict__ out, float2* __restrict__ coef,
                                                                    const ga_delta_args a,
-                                                                   const int32_t* __restrict__ token_entry, int tokens) {
+                                                                   const int32_t* __restrict__ token_entry, int tokens, int logs) {
   __shared__ float ys[TB][DL_THREADS];
   __shared__ float factor[TB][DL_THREADS];
   const int tid = threadIdx.x;
@@ -140,7 +101,9 @@ __global__ __launch_bounds__(DL_THREADS) void delta_prepare_kernel(float* __rest
       const int64_t t = t0 + i / a.heads;
       const int h = i % a.heads;
       const float* row = a.proj + t * a.stride;
-      coef[t * a.heads + h] = dl_coefficients(a.delta, row[a.a_at + h], row[a.b_at + h], a.dt_bias[h], a.rate[h]);
+      float2 c2 = dl_log_coefficients(a.delta, row[a.a_at + h], row[a.b_at + h], a.dt_bias[h], a.rate[h]);
+      if (!logs) c2.x = expf(c2.x);
+      coef[t * a.heads + h] = c2;
     }
     return;
   }
@@ -376,13 +339,7 @@ __global__ __launch_bounds__(DL_THREADS) __attribute__((amdgpu_waves_per_eu(1, 4
 #pragma unroll
       for (int j = 0; j < R4; ++j) st[(c * R4 + j) * WAVE] = S[c][j];
     }
-  // the last taps inputs of the entry into the ring, the channels dealt to the entry's workgroups
-  if (a.taps > 1) {
-    const int per = gridDim.y * gridDim.z * DL_THREADS, mine = (h * gridDim.z + blockIdx.z) * DL_THREADS + tid;
-    for (int c = mine; c < a.channels; c += per)
-      for (int i = max(0, n - a.taps); i < n; ++i)
-        a.ring[(slot * a.taps + (start + i) % a.taps) * (int64_t)a.channels + c] = a.proj[(int64_t)(first + i) * a.stride + a.conv_at + c];
-  }
+  dl_keep_inputs(a, first, n, start, slot, (h * gridDim.z + blockIdx.z) * DL_THREADS + tid, gridDim.y * gridDim.z * DL_THREADS);
 }
 
 // ---------------------------------------------------------------------------------------------------- step
@@ -477,7 +434,8 @@ __global__ __launch_bounds__(DL_THREADS) void delta_step_kernel(T* __restrict__ 
       else vs[i - 2 * a.dim] = y;
     }
   }
-  const float2 c2 = dl_coefficients(DELTA, za, zb, dt_bias, rate);
+  float2 c2 = dl_log_coefficients(DELTA, za, zb, dt_bias, rate);
+  c2.x = expf(c2.x);
   __syncthreads();
   if (DELTA) {
     if (wave < 2) {
@@ -532,17 +490,10 @@ __global__ __launch_bounds__(DL_THREADS) void delta_step_kernel(T* __restrict__ 
   }
 }
 
-static int dl_check(const ga_delta_args& a) {
-  if (a.heads <= 0 || a.groups <= 0 || a.heads % a.groups || a.dim <= 0 || a.dim > 256 || a.vdim <= 0 || a.vdim > DL_MAX_VDIM) return -1;
-  if (a.taps < 1 || a.taps > DL_MAX_TAPS || (a.taps > 1 && !a.ring) || !a.conv_w) return -2;
-  if (a.heads > 65535) return -3;
-  if (!a.proj || !a.state || !a.slots || !a.cu || !a.q_start || !a.rate || !a.dt_bias || (!a.delta && !a.skip)) return -4;
-  return 0;
-}
-
 extern "C" int64_t ga_delta_row(const ga_delta_args* args) { return dl_row(*args); }
 
-extern "C" int ga_delta_prepare(void* act, void* coef, const ga_delta_args* args, const void* token_entry, int tokens, hipStream_t stream) {
+extern "C" int ga_delta_prepare(void* act, void* coef, const ga_delta_args* args, const void* token_entry, int tokens, int logs,
+                                hipStream_t stream) {
   if (tokens <= 0) return 0;
   const ga_delta_args& a = *args;
   const int rc = dl_check(a);
@@ -552,7 +503,7 @@ extern "C" int ga_delta_prepare(void* act, void* coef, const ga_delta_args* args
   const int64_t blocks = (units + heads_here - 1) / heads_here + (plain + DL_THREADS - 1) / DL_THREADS + 1;
   if (plain < 0 || blocks > 65535 || dl_row(a) > (1 << 26)) return -5;
 #define GO(TAPS, TB) hipLaunchKernelGGL((delta_prepare_kernel<TAPS, TB>), dim3((tokens + TB - 1) / TB, (unsigned)blocks), dim3(DL_THREADS), 0, \
-                                        stream, (float*)act, (float2*)coef, a, (const int32_t*)token_entry, tokens)
+                                        stream, (float*)act, (float2*)coef, a, (const int32_t*)token_entry, tokens, logs)
   const bool few = (int64_t)tokens * blocks <= 2048;         // a token to a workgroup while that does not fill the chip
   if (a.taps == 4) { if (few) GO(4, 1); else GO(4, DL_PREP_TOKENS); }
   else { if (few) GO(0, 1); else GO(0, DL_PREP_TOKENS); }

@@ -339,15 +339,25 @@ typedef struct {
   float q_scale, unit_eps;
 } ga_delta_args;
 // act float [tokens, ga_delta_row(args)]: the channels convolved, silu, q and k (delta) as unit vectors, q times q_scale, as the
-// scan reads them (16-byte aligned); coef float [tokens, heads, 2]: decays and steps
+// scan reads them (16-byte aligned); coef float [tokens, heads, 2]: decays (logs: their logarithms) and steps
 int64_t ga_delta_row(const ga_delta_args* args);
-int ga_delta_prepare(void* act, void* coef, const ga_delta_args* args, const void* token_entry, int tokens, hipStream_t stream);
+int ga_delta_prepare(void* act, void* coef, const ga_delta_args* args, const void* token_entry, int tokens, int logs,
+                     hipStream_t stream);
 // out float [tokens, heads, vdim]: o (delta), or (o + skip v) silu(gate); advances state and ring
 int ga_delta_scan(void* out, const void* act, const void* coef, const ga_delta_args* args, int entries, hipStream_t stream);
 // every entry brings one token: all of it in one launch; delta: out (compute dtype, row stride out_stride) = out_scale * weight *
 // silu(gate) * o / rms(o), else float, as the scan's
 int ga_delta_step(void* out, int64_t out_stride, const ga_delta_args* args, const void* weight, float eps, float out_scale,
                   int out_bf16, int entries, hipStream_t stream);
+
+// ---- delta_chunk.hip: the scan of delta_scan.hip in chunks of 16 tokens on the matrix cores (32-bit products).  plan: from act and
+// coef (with logs) the operands of every chunk: ops and heads float, 16-byte aligned, of ga_delta_chunk_floats (what 0 / 1)
+// elements; scan: state and ring as ga_delta_scan's, out too, with a row behind the last token's (which holds anything)
+int64_t ga_delta_chunk_floats(const ga_delta_args* args, int tokens, int entries, int what);
+int ga_delta_chunk_plan(void* ops, void* heads, const void* act, const void* coef, const ga_delta_args* args, int tokens, int entries,
+                        hipStream_t stream);
+int ga_delta_chunk_scan(void* out, const void* ops, const void* heads, const void* act, const ga_delta_args* args, int tokens, int entries,
+                        hipStream_t stream);
 
 // ---- pooled_attention.hip: attention over a window of tokens and the means of the blocks before it, sigmoid weights.
 // prepare: q and k of a 32-bit projection [q heads | k heads | v heads ...] turned by position (pairs 2i, 2i + 1), divided by

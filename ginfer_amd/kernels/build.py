@@ -26,11 +26,11 @@ FLAGS = ["--offload-arch=" + ARCH, "-O3", "-std=c++17", "-shared", "-fPIC",
 MODULES = ("embedding", "norm", "rope_kv", "attention_generic", "attention_mfma", "gemm", "gemm_skinny",
            "activation", "sampling", "random_fill", "scalar_norm", "embedding_sinusoid", "short_conv", "gated_recurrence",
            "latent_attention", "output_norm", "routing", "conv_rope_kv", "decay_scan", "pooled_attention",
-           "gated_residual", "hyper_connection", "rglru", "layer_norm", "expert_gemm", "delta_scan")
+           "gated_residual", "hyper_connection", "rglru", "layer_norm", "expert_gemm", "delta_scan", "delta_chunk")
 # flags of single modules: the random-weights generator must round every operation by itself, as the host's twin does
 MODULE_FLAGS = {"random_fill": ["-ffp-contract=off"], "attention_generic": ["-ffp-contract=off"]}
 # headers beside common.h that a module includes (they enter its digest)
-MODULE_HEADERS = {"random_fill": ["random_normal.h"]}
+MODULE_HEADERS = {"random_fill": ["random_normal.h"], "delta_scan": ["delta_common.h"], "delta_chunk": ["delta_common.h"]}
 # plain C++ libraries for the host (no GPU runtime), built with the host compiler from csrc/host/
 HOST_MODULES = ("random_fill_host",)
 HOST_FLAGS = ["-O2", "-std=c++17", "-shared", "-fPIC", "-pthread", "-ffp-contract=off"]

@@ -1694,14 +1694,18 @@ def delta_state_matrix(state, dim, vdim):
 
 
 def delta_recurrence(proj, conv_weight, conv_bias, rate, dt_bias, skip, ring, state, slots, step, heads, groups, dim, vdim, columns, delta,
-                     q_scale=1.0, unit_eps=0.0, weight=None, eps=0.0, dtype=None, out=None, out_scale=1.0):
+                     q_scale=1.0, unit_eps=0.0, weight=None, eps=0.0, dtype=None, out=None, out_scale=1.0,
+                     chunked=False):
     """One step of the recurrence (csrc/delta_scan.hip has the equations) over per-request state.  proj: float32 [T, ..] rows with
     unit inner stride; `columns` names where its parts begin: conv (the convolved channels), a and b (the decay's and the
     step's numbers per head), gate [heads * vdim], and, among the convolved channels, q, k and v.  conv_weight float32 [channels,
     taps], conv_bias float32 [channels] or None; rate, dt_bias float32 [heads]; ring float32 [slots, taps, channels] (None for
     one tap) and state float32 [slots, *delta_state_shape] are advanced in place.
     delta: returns [T, heads * vdim] in `dtype`: out_scale * weight * silu(gate) * o / rms(o) per head (weight float32 [vdim]),
-    into `out` where it is given.  Else: float32 [T, heads, vdim]: (o + skip v) silu(gate), skip float32 [heads]."""
+    into `out` where it is given.  Else: float32 [T, heads, vdim]: (o + skip v) silu(gate), skip float32 [heads].
+    Without `chunked` every token's sums are taken in an order of their own, so the bits do not depend on how the tokens were cut
+    into steps; chunked: prompt portions go in chunks of 16 tokens over the matrix cores (csrc/delta_chunk.hip; 32-bit operands
+    and sums), and results differ by rounding with the cut."""
     _dev(proj, conv_weight, conv_bias, rate, dt_bias, skip, ring, state, slots, weight, out)
     T = proj.shape[0]
     _need(proj.dtype == torch.float32 and proj.dim() == 2 and proj.stride(1) == 1, "proj must be float32 [T, ..] with unit inner stride")
@@ -1758,9 +1762,21 @@ def delta_recurrence(proj, conv_weight, conv_bias, rate, dt_bias, skip, ring, st
     lib.ga_delta_row.restype = ctypes.c_int64
     act = torch.empty((T, lib.ga_delta_row(ctypes.byref(args))), dtype=torch.float32, device=proj.device)
     coef = torch.empty((T, heads, 2), dtype=torch.float32, device=proj.device)
-    o = torch.empty((T, heads, vdim), dtype=torch.float32, device=proj.device)
-    _check(lib.ga_delta_prepare(_ptr(act), _ptr(coef), ctypes.byref(args), _ptr(step.token_entry), _i(T), _stream()), "delta_prepare")
-    _check(lib.ga_delta_scan(_ptr(o), _ptr(act), _ptr(coef), ctypes.byref(args), _i(E), _stream()), "delta_scan")
+    # (the kernel in chunks stores what is no token's into a row of its own)
+    o = torch.empty((T + 1, heads, vdim), dtype=torch.float32, device=proj.device)[:T]
+    _check(lib.ga_delta_prepare(_ptr(act), _ptr(coef), ctypes.byref(args), _ptr(step.token_entry), _i(T), _i(1 if chunked else 0),
+                                _stream()), "delta_prepare")
+    if chunked:
+        lib = build.load("delta_chunk")
+        lib.ga_delta_chunk_floats.restype = ctypes.c_int64
+        operands, per_head = (torch.empty((lib.ga_delta_chunk_floats(ctypes.byref(args), _i(T), _i(E), _i(what)),), dtype=torch.float32,
+                                          device=proj.device) for what in (0, 1))
+        _check(lib.ga_delta_chunk_plan(_ptr(operands), _ptr(per_head), _ptr(act), _ptr(coef), ctypes.byref(args), _i(T), _i(E), _stream()),
+               "delta_chunk_plan")
+        _check(lib.ga_delta_chunk_scan(_ptr(o), _ptr(operands), _ptr(per_head), _ptr(act), ctypes.byref(args), _i(T), _i(E), _stream()),
+               "delta_chunk_scan")
+    else:
+        _check(lib.ga_delta_scan(_ptr(o), _ptr(act), _ptr(coef), ctypes.byref(args), _i(E), _stream()), "delta_scan")
     if not delta:
         return o
     return head_norm_gate(o, weight, eps, dtype, proj=proj, gate_start=at["gate"], out=out, out_scale=out_scale)

@@ -36,12 +36,12 @@ class _DeltaMixer(Part):
         return [StateSpec(ops.delta_state_shape(self.nh, self.dk, self.dv), torch.float32), ring]
 
     def kernel_modules(self):
-        return ["delta_scan", "decay_scan", "gemm"] + (["gemm_skinny"] if self.dtype == torch.bfloat16 else [])
+        return ["delta_scan", "decay_scan", "gemm"] + (["delta_chunk", "gemm_skinny"] if self.dtype == torch.bfloat16 else [])
 
     def _recurrence(self, proj, step, cache, **kw):
         state, ring = cache
         return ops.delta_recurrence(proj, self.w_conv, self.b_conv, self.rate, self.dt_bias, self.skip, None if ring is None else ring.state,
-                                    state.state, state.slots, step, self.nh, self.ng, self.dk, self.dv, self.columns, **kw)
+                                    state.state, state.slots, step, self.nh, self.ng, self.dk, self.dv, self.columns, chunked=self.dtype == torch.bfloat16, **kw)
 
     # (what `ParallelSum` needs to share the two products: see ConvAttention)
     @property

@@ -194,13 +194,14 @@ def test_head_norms_with_gates(dtype):
 CUTS = [None, [1, 1, 2, 5, 3, 16, 1, 17, 1, 64, 24, 15], [2] * 75, [1] * 150]
 
 
+@pytest.mark.parametrize("chunked", [False, True])
 @pytest.mark.parametrize("delta", [True, False])
 @pytest.mark.parametrize("sizes", [(1, 1, 64, 4, 4), (6, 3, 8, 12, 3), (2, 2, 20, 7, 4), (5, 1, 33, 20, 1), (4, 2, 130, 64, 4), (9, 3, 17, 5, 6),
                                    (2, 1, 250, 40, 4), (3, 3, 128, 130, 2), (1, 1, 1, 1, 16), (4, 1, 192, 260, 4)])
-def test_the_recurrences_alone(delta, sizes):
+def test_the_recurrences_alone(delta, sizes, chunked):
     """Whole, cut in several ways and token by token, beside a second request that starts and ends elsewhere, against the plain
     statement; the state is the plain one; slots that held something else (here: no numbers at all) show nowhere; all cuttings give
-    the same bits."""
+    the same bits, or, in chunks on the matrix cores, the same up to rounding."""
     from ginfer_amd.kernels import ops
     heads, groups, dim, vdim, taps = sizes
     g = torch.Generator().manual_seed(sum(sizes))
@@ -255,7 +256,7 @@ def test_the_recurrences_alone(delta, sizes):
             slots = torch.tensor([e[0] for e in entries], device="cuda")
             out = ops.delta_recurrence(rows, dev(w), dev(bias), dev(rate), dev(dt), dev(skip), ring, state, slots, step, heads, groups, dim, vdim,
                                        cols, delta, q_scale=dim ** -0.5, unit_eps=1e-6, weight=dev(weight) if delta else None, eps=1e-5,
-                                       dtype=torch.float32, out_scale=0.7).cpu()
+                                       dtype=torch.float32, out_scale=0.7, chunked=chunked).cpu()
             mine = (k if i % 2 and k else 0)
             got.append(out[mine:mine + n])
             if k:
@@ -268,6 +269,8 @@ def test_the_recurrences_alone(delta, sizes):
         held = ops.delta_state_matrix(state[2].cpu(), dim, vdim)
         assert H.rel_err(held, S_want) < 2e-5
         first = first or (got, held)
+        if chunked:
+            continue
         assert torch.equal(got, first[0]) and torch.equal(held, first[1]), "%d steps differ from one" % len(cut)
 
 
@@ -290,10 +293,10 @@ def test_an_old_write_reaches_far_and_slow_decay_counts():
     proj[-1, :dim] = -30.0
     proj[-1, 2] = 8.0                                # and the query that asks for it
     w = torch.ones((C, 1))
-    args = lambda rows, state, step: ops.delta_recurrence(
+    args = lambda rows, state, step, chunked: ops.delta_recurrence(
         rows.cuda(), w.cuda(), None, torch.ones(1, device="cuda"), torch.zeros(1, device="cuda"), None, None, state,
         torch.zeros(1, dtype=torch.int64, device="cuda"), step, 1, 1, dim, vdim, cols, True, q_scale=dim ** -0.5, unit_eps=1e-6,
-        weight=torch.ones(vdim, device="cuda"), eps=1e-5, dtype=torch.float32)
+        weight=torch.ones(vdim, device="cuda"), eps=1e-5, dtype=torch.float32, chunked=chunked)
     c = pp.silu(proj[:, :C].double())
     q, k, v = pp.unit(c[:, :dim])[:, None] * dim ** -0.5, pp.unit(c[:, dim:2 * dim])[:, None], c[:, 2 * dim:][:, None]
     a, b = torch.exp(-pp.softplus(proj[:, cols["a"]:cols["a"] + 1].double())), torch.sigmoid(proj[:, cols["b"]:cols["b"] + 1].double())
@@ -301,13 +304,40 @@ def test_an_old_write_reaches_far_and_slow_decay_counts():
     want = pp.rms(o[-1, 0], 1e-5) * pp.silu(torch.tensor(2.0, dtype=torch.float64))
     gone = pp.rms(pp.gated_delta_rule(q[16:], k[16:], v[16:], a[16:], b[16:])[0][-1, 0], 1e-5) * pp.silu(torch.tensor(2.0, dtype=torch.float64))
     assert H.rel_err(gone, want) > 0.3
-    for cut in ([720], [16, 1, 700, 3], [700] + [1] * 20):
+    for cut, chunked in [(c, k) for c in ([720], [16, 1, 700, 3], [700] + [1] * 20) for k in (False, True)]:
         state = torch.zeros((1,) + ops.delta_state_shape(1, dim, vdim), device="cuda")
         at = 0
         for n in cut:
-            out = args(proj[at:at + n], state, _Step([n], [at]))
+            out = args(proj[at:at + n], state, _Step([n], [at]), chunked)
             at += n
         assert H.rel_err(out[-1].cpu(), want) < 5e-5
+
+
+@pytest.mark.parametrize("chunked", [False, True])
+def test_the_same_key_again_and_again(chunked):
+    """Every token writes under the same key with b near 1 and no decay to speak of: each write overwrites the one before, and what
+    is read is the last value.  Inside a chunk the writes then cancel to first order, which a product of powers would lose."""
+    from ginfer_amd.kernels import ops
+    T, dim, vdim = 100, 64, 32
+    g = torch.Generator().manual_seed(4)
+    C = 2 * dim + vdim
+    cols = dict(conv=0, q=0, k=dim, v=2 * dim, gate=C, b=C + vdim, a=C + vdim + 1)
+    proj = torch.zeros((T, C + vdim + 2))
+    proj[:, :2 * dim] = torch.randn((2 * dim,), generator=g)
+    proj[:, 2 * dim:C] = torch.randn((T, vdim), generator=g) * 3
+    proj[:, C:C + vdim] = 1.5
+    proj[:, cols["b"]], proj[:, cols["a"]] = 12.0, -12.0
+    proj[:, :dim] = proj[:, dim:2 * dim]
+    state = torch.zeros((1,) + ops.delta_state_shape(1, dim, vdim), device="cuda")
+    out = ops.delta_recurrence(proj.cuda(), torch.ones((C, 1), device="cuda"), None, torch.ones(1, device="cuda"), torch.zeros(1, device="cuda"), None,
+                               None, state, torch.zeros(1, dtype=torch.int64, device="cuda"), _Step([T], [0]), 1, 1, dim, vdim, cols, True,
+                               q_scale=dim ** -0.5, unit_eps=1e-6, weight=torch.ones(vdim, device="cuda"), eps=0.0, dtype=torch.float32, chunked=chunked)
+    want = pp.rms(pp.silu(proj[:, 2 * dim:C].double()), 0.0) * pp.silu(torch.tensor(1.5, dtype=torch.float64))
+    assert H.rel_err(out.cpu(), want) < 1e-3
+    c = pp.silu(proj[:, :C].double())
+    o, _ = pp.gated_delta_rule(pp.unit(c[:, None, :dim]) * dim ** -0.5, pp.unit(c[:, None, dim:2 * dim]), c[:, None, 2 * dim:],
+                               torch.exp(-pp.softplus(proj[:, cols["a"]:cols["a"] + 1].double())), torch.sigmoid(proj[:, cols["b"]:cols["b"] + 1].double()))
+    assert H.rel_err(out.cpu(), pp.rms(o[:, 0], 0.0) * pp.silu(torch.tensor(1.5, dtype=torch.float64))) < 2e-5
 
 
 @pytest.mark.parametrize("experts,identity,top", [(1, 0, 1), (6, 2, 2), (5, 3, 8), (60, 4, 6), (200, 56, 8), (3, 1, 1)])
