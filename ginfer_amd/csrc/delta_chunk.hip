@@ -296,7 +296,7 @@ __global__ __launch_bounds__(DL_THREADS) __attribute__((amdgpu_waves_per_eu(2, 4
       S[j] = R[j];
       asm volatile("" : "+v"(S[j]));
     }
-    asm volatile("s_nop 15");
+    asm volatile("s_nop 15");                              // the next chunk, behind a branch, may read S in its first instruction
   };
   for (int c = 0; c < chunks; c += 6) {
     chunk(c, x[0], x[2], 0);
